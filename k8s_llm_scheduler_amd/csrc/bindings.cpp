@@ -117,7 +117,10 @@ int k8s_embed_rows(float* out, const int* ids, const void* table, int T, int W, 
 int k8s_resnorm(float* x, const void* branch, const void* branch2, float mult, const void* rowvec, const void* w,
                 float offset, float eps, void* out, int T, int W, int groups, int f32, hipStream_t s);
 int k8s_norm_mix(void* out, const void* a, long lda, const void* wa, const void* b, const void* wb, float eps, float ca,
-                 float cb, int T, int W, int groups, int in_f32, int out_f32, hipStream_t s);
+                 float cb, int T, int W, int groups, const void* gate, long ldg, int gkind, int in_f32, int out_f32,
+                 hipStream_t s);
+int k8s_branchnorm(float* x, const void* branch, const void* w, float eps, void* out, int T, int W, int branch_f32,
+                   int f32, hipStream_t s);
 int k8s_postnorm(float* x, const void* branch, const void* branch2, float alpha, float c1, float c2, float gain,
                  float eps, void* out, int T, int W, int f32, hipStream_t s);
 int k8s_gate_mul(void* out, const void* y, long ldy, const void* gate, long ldg, int T, int F, int kind, int y_f32,
@@ -156,12 +159,13 @@ int k8s_latent_kv_write(void* cache, const void* dkv, const void* normw, void* q
                         float eps, int f32, long ldd, int interleaved, hipStream_t s);
 int k8s_latent_attention(void* out, const void* q_abs, const void* q, const void* cache, const int* block_tables,
                          int max_blocks, const int* tok_seq, const int* positions, int T, int C, int R, int H, int Dn,
-                         int window, float scale, int bs, int f32, const float* sinks, hipStream_t s);
+                         int window, float scale, int bs, int f32, const float* sinks, const void* gate, long ldg,
+                         hipStream_t s);
 int k8s_latent_mfma_ok(int C, int R, int Dn);
 int k8s_latent_attention_mfma(void* out, float* pacc, float* pml, const void* q_abs, const void* q, const void* cache,
                               const int* block_tables, int max_blocks, const int* tok_seq, const int* positions, int T,
                               int C, int R, int H, int Dn, int window, float scale, int bs, int nsplit, const int* cu_q,
-                              int nseq, int max_qlen, const float* sinks, hipStream_t s);
+                              int nseq, int max_qlen, const float* sinks, const void* gate, long ldg, hipStream_t s);
 int k8s_moe_route(int* idx, float* w, const float* logits, int ld, int T, int E, int top, float scale, int mode,
                   hipStream_t s);
 int k8s_window_kv_write(void* kcache, void* vcache, void* qkv, long ld, int koff, int voff, const void* qb,
@@ -186,7 +190,7 @@ int k8s_window_attention_mfma(void* out, const void* q, long ldq, const void* ga
                               const float* sinkv, int gate_ph, hipStream_t s);
 int k8s_gated_scan_max_dim();
 long long k8s_gated_scan_record(int kind, int D, int V);
-int k8s_gated_scan(void* out, const float* proj, long ld, int kind, int cq, int ck, int cv, int ci, int cf, int cg,
+int k8s_gated_scan(void* out, const void* proj, long ld, int kind, int cq, int ck, int cv, int ci, int cf, int cg,
                    const void* fbias, const void* ibias, const void* lower, const void* normw, float* state,
                    const int* cu_q, const int* seq_slots, const int* positions, int nseq, int H, int D, int V, float eps,
                    float cap, int f32, int T, int Lc, float* ws, const float* aux, long ldaux, const float* hpar, int R,
@@ -463,9 +467,14 @@ PYBIND11_MODULE(K8S_MODULE_NAME, m) {
                       S(s)), "resnorm");
   });
   m.def("norm_mix", [](uintptr_t out, uintptr_t a, long lda, uintptr_t wa, uintptr_t b, uintptr_t wb, float eps,
-                       float ca, float cb, int T, int W, int groups, int in_f32, int out_f32, int64_t s) {
-    check(k8s_norm_mix(P(out), P(a), lda, P(wa), P(b), P(wb), eps, ca, cb, T, W, groups, in_f32, out_f32, S(s)),
-          "norm_mix");
+                       float ca, float cb, int T, int W, int groups, uintptr_t gate, long ldg, int gkind, int in_f32,
+                       int out_f32, int64_t s) {
+    check(k8s_norm_mix(P(out), P(a), lda, P(wa), P(b), P(wb), eps, ca, cb, T, W, groups, P(gate), ldg, gkind, in_f32,
+                       out_f32, S(s)), "norm_mix");
+  });
+  m.def("branchnorm", [](uintptr_t x, uintptr_t branch, uintptr_t w, float eps, uintptr_t out, int T, int W,
+                         int branch_f32, int f32, int64_t s) {
+    check(k8s_branchnorm(P<float>(x), P(branch), P(w), eps, P(out), T, W, branch_f32, f32, S(s)), "branchnorm");
   });
   m.def("postnorm", [](uintptr_t x, uintptr_t branch, uintptr_t branch2, float alpha, float c1, float c2, float gain,
                        float eps, uintptr_t out, int T, int W, int f32, int64_t s) {
@@ -544,9 +553,11 @@ PYBIND11_MODULE(K8S_MODULE_NAME, m) {
   });
   m.def("latent_attention", [](uintptr_t out, uintptr_t q_abs, uintptr_t q, uintptr_t cache, uintptr_t bt,
                                int max_blocks, uintptr_t tok_seq, uintptr_t positions, int T, int C, int R, int H,
-                               int Dn, int window, float scale, int bs, int f32, uintptr_t sinks, int64_t s) {
+                               int Dn, int window, float scale, int bs, int f32, uintptr_t sinks, uintptr_t gate, long ldg,
+                               int64_t s) {
     check(k8s_latent_attention(P(out), P(q_abs), P(q), P(cache), P<int>(bt), max_blocks, P<int>(tok_seq),
-                               P<int>(positions), T, C, R, H, Dn, window, scale, bs, f32, P<float>(sinks), S(s)),
+                               P<int>(positions), T, C, R, H, Dn, window, scale, bs, f32, P<float>(sinks), P(gate), ldg,
+                               S(s)),
           "latent_attention");
   });
   m.def("latent_mfma_ok", [](int C, int R, int Dn) { return k8s_latent_mfma_ok(C, R, Dn) != 0; });
@@ -554,10 +565,10 @@ PYBIND11_MODULE(K8S_MODULE_NAME, m) {
                                     uintptr_t cache, uintptr_t bt, int max_blocks, uintptr_t tok_seq,
                                     uintptr_t positions, int T, int C, int R, int H, int Dn, int window, float scale,
                                     int bs, int nsplit, uintptr_t cu_q, int nseq, int max_qlen, uintptr_t sinks,
-                                    int64_t s) {
+                                    uintptr_t gate, long ldg, int64_t s) {
     check(k8s_latent_attention_mfma(P(out), P<float>(pacc), P<float>(pml), P(q_abs), P(q), P(cache), P<int>(bt),
                                     max_blocks, P<int>(tok_seq), P<int>(positions), T, C, R, H, Dn, window, scale, bs,
-                                    nsplit, P<int>(cu_q), nseq, max_qlen, P<float>(sinks), S(s)),
+                                    nsplit, P<int>(cu_q), nseq, max_qlen, P<float>(sinks), P(gate), ldg, S(s)),
           "latent_attention_mfma");
   });
   m.def("moe_route", [](uintptr_t idx, uintptr_t w, uintptr_t logits, int ld, int T, int E, int top, float scale,
@@ -612,7 +623,7 @@ PYBIND11_MODULE(K8S_MODULE_NAME, m) {
                          uintptr_t cu_q, uintptr_t seq_slots, uintptr_t positions, int nseq, int H, int D, int V,
                          float eps, float cap, int f32, int T, int Lc, uintptr_t ws, uintptr_t aux, long ldaux,
                          uintptr_t hpar, int R, int64_t s) {
-    check(k8s_gated_scan(P(out), P<float>(proj), ld, kind, cq, ck, cv, ci, cf, cg, P(fbias), P(ibias), P(lower),
+    check(k8s_gated_scan(P(out), P(proj), ld, kind, cq, ck, cv, ci, cf, cg, P(fbias), P(ibias), P(lower),
                          P(normw), P<float>(state), P<int>(cu_q), P<int>(seq_slots), P<int>(positions), nseq, H, D, V,
                          eps, cap, f32, T, Lc, P<float>(ws), P<float>(aux), ldaux, P<float>(hpar), R, S(s)),
           "gated_scan");

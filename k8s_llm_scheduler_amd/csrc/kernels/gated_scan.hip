@@ -13,10 +13,18 @@
 //       no norm here (it runs over groups of heads afterwards) and y is stored in fp32.  x, B and C come from `proj`
 //       (the convolved branch), zdt and zg from `aux` (the input projection); neg_a, dt_bias and skip from `hpar`
 //       ([3][H] fp32).
+//   KIND 3 (linear attention with a constant decay per head, "lightning")
+//       q = silu(zq), k = silu(zk), v = silu(zv);  S <- a S + k v^T with a = hpar[head] in (0, 1];  o = S^T q, stored in
+//       fp32 (the norm over all heads and the gate follow in another kernel); q and k [D] are shared by the R heads of a
+//       group, v [V] is the head's own.  The projected row is read in the activation type: nothing but projections and
+//       their activations enters this recurrence.
 // Everything that enters the recurrence (gates, decays, state, norms) is fp32: the kernels read the fused input
-// projection as fp32 [T, ld] with the parts at column offsets, and write y in the activation type.
+// projection as fp32 [T, ld] (KIND 3: activation type) with the parts at column offsets, and write y in the activation
+// type (KIND 2, 3: fp32).
 // Varlen batches: sequence s owns tokens cu_q[s] .. cu_q[s + 1] - 1 and the state record of slot seq_slots[s]; a portion
 // that starts at position 0 starts from zero state (m = 0), so a reused slot needs no clearing.
+#include <type_traits>
+
 #include "common.h"
 
 namespace k8sllm {
@@ -27,7 +35,7 @@ struct ScanCols { int q, k, v, i, f, g; };   // column offsets of the parts insi
 // [c CH, (c + 1) CH) of S; group c = 0 prepares each token's per-channel read / keep / write coefficients in LDS (and,
 // KIND 1, owns n).  The partial outputs of the channel groups meet in LDS; group 0 normalises and stores.  The next
 // token's inputs are loaded while the current one is computed; the barriers wait for LDS traffic only.
-// blockDim = (DX, NS): DX = max(D, V) (KIND 2: V) rounded up to 64, NS = ceil(D / CH), CH (16, 32 or 64) the smallest
+// blockDim = (DX, NS): DX = max(D, V) (KIND 2, 3: V) rounded up to 64, NS = ceil(D / CH), CH (16, 32 or 64) the smallest
 // that keeps DX NS within 1024 threads.  State record: S [D][V] (, n [D], m).
 //
 // MODE 0: a whole portion per workgroup, from the slot's state (zero at position 0) to the slot's state.
@@ -40,8 +48,12 @@ struct ScanCols { int q, k, v, i, f, g; };   // column offsets of the parts insi
 //           KIND 0: start[c + 1] = dec[c] * start[c] + loc[c]
 //           KIND 1: m' = max(F + m, m_loc); (S, n)[c + 1] = e^(F + m - m') (S, n)[c] + e^(m_loc - m') (S, n)_loc
 // MODE 2: a chunk from its start state with outputs; a sequence's last chunk leaves the slot's state.
+template <typename TA, int KIND> using scan_in_t = std::conditional_t<KIND == 3, TA, float>;
+__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
+
 template <typename TA, int CH, int KIND, int MODE>
-__global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out, const float* __restrict__ proj, long ld,
+__global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out,
+                                                          const scan_in_t<TA, KIND>* __restrict__ proj, long ld,
                                                           ScanCols co, const TA* __restrict__ fbias,
                                                           const TA* __restrict__ ibias, const TA* __restrict__ lower,
                                                           const TA* __restrict__ normw, float* __restrict__ state,
@@ -81,10 +93,10 @@ __global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out, 
   }
   const int x = threadIdx.x, c = threadIdx.y, NS = blockDim.y, DX = blockDim.x;
   const bool onv = x < V, ond = x < D;
-  // KIND 2: the block is as wide as the value columns only, and the D shared inputs of a token (B, C) are loaded by the
+  // KIND 2, 3: the block is as wide as the value columns only, and the D shared inputs of a token are loaded by the
   // first ceil(D / DX) thread groups, element c DX + x each
   const int le = c * DX + x;
-  const bool ldr = KIND == 2 && le < D;
+  const bool ldr = KIND >= 2 && le < D;
   const int i0 = c * CH;
   const size_t rec = (size_t)D * V + (KIND == 1 ? D + 1 : 0);       // slot record
   const size_t crec = (size_t)D * V + D + 2;                         // chunk record
@@ -107,8 +119,10 @@ __global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out, 
     for (int e = x; e < DMAX; e += DX) sq[e] = sa[e] = sb[e] = 0.f;
   float lowx = 0.f, fbx = 0.f, nwx = 0.f, fbh = 0.f, ibh = 0.f;
   float nega = 0.f, skip = 0.f;
-  const int qk0 = KIND == 2 ? (hd / R) * D : hd * D;    // the head's (KIND 2: its group's) query / key columns
-  if (KIND == 2) {
+  const int qk0 = KIND >= 2 ? (hd / R) * D : hd * D;    // the head's (KIND 2, 3: its group's) query / key columns
+  if (KIND == 3) {
+    nega = hpar[hd];                 // the decay itself
+  } else if (KIND == 2) {
     nega = hpar[hd];
     fbh = hpar[H + hd];
     skip = hpar[2 * H + hd];
@@ -129,35 +143,48 @@ __global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out, 
   float nq = 0.f, nk = 0.f, nv = 0.f, nf = 0.f, ni = 0.f, ng = 0.f;
   auto fetch = [&](int t) {
     if (t >= b0) return;
-    const float* r = proj + (size_t)t * ld;
-    if (onv) nv = r[co.v + (size_t)hd * V + x];
+    const scan_in_t<TA, KIND>* r = proj + (size_t)t * ld;
+    if (onv) nv = ldf(r, co.v + (size_t)hd * V + x);
+    if (KIND == 3) {
+      if (ldr) {
+        if (MODE != 1) nq = ldf(r, co.q + qk0 + le);
+        nk = ldf(r, co.k + qk0 + le);
+      }
+      return;
+    }
     if (KIND == 2) {
       const float* ar = aux + (size_t)t * ldaux;
       nf = ar[co.f + hd];
       if (MODE != 1 && c == 0 && onv) ng = ar[co.g + (size_t)hd * V + x];
       if (ldr) {
-        if (MODE != 1) nq = r[co.q + qk0 + le];
-        nk = r[co.k + qk0 + le];
+        if (MODE != 1) nq = ldf(r, co.q + qk0 + le);
+        nk = ldf(r, co.k + qk0 + le);
       }
       return;
     }
     if (KIND == 1) {
-      nf = r[co.f + hd];
-      ni = r[co.i + hd];
-      if (MODE != 1 && c == 0 && onv) ng = r[co.g + (size_t)hd * V + x];
+      nf = ldf(r, co.f + hd);
+      ni = ldf(r, co.i + hd);
+      if (MODE != 1 && c == 0 && onv) ng = ldf(r, co.g + (size_t)hd * V + x);
     }
     if (c == 0 && ond) {
-      if (MODE != 1) nq = r[co.q + (size_t)hd * D + x];
-      if (KIND == 0) nf = r[co.f + (size_t)hd * D + x];
-      else nk = r[co.k + (size_t)hd * D + x];
+      if (MODE != 1) nq = ldf(r, co.q + (size_t)hd * D + x);
+      if (KIND == 0) nf = ldf(r, co.f + (size_t)hd * D + x);
+      else nk = ldf(r, co.k + (size_t)hd * D + x);
     }
   };
   fetch(a0);
   for (int t = a0; t < b0; ++t) {
-    const float cq = nq, ck = nk, cv = nv, cf = nf, ci = ni, cg = ng;
+    const float cq = nq, ck = nk, cv = KIND == 3 ? silu_f(nv) : nv, cf = nf, ci = ni, cg = ng;
     fetch(t + 1);
-    float ka = 1.f;   // KIND 1, 2: the head's keep factor
-    if (KIND == 2) {
+    float ka = 1.f;   // KIND 1, 2, 3: the head's keep factor
+    if (KIND == 3) {
+      ka = nega;
+      if (ldr) {
+        sq[le] = silu_f(cq);
+        sb[le] = silu_f(ck);
+      }
+    } else if (KIND == 2) {
       const float zd = cf + fbh;
       const float dt = fmaxf(zd, 0.f) + log1pf(expf(-fabsf(zd)));
       ka = expf(nega * dt);
@@ -218,11 +245,11 @@ __global__ __launch_bounds__(1024) void gated_scan_kernel(TA* __restrict__ out, 
     if (onv) po[c][x] = (o4[0] + o4[1]) + (o4[2] + o4[3]);
     lds_barrier();
     float o = 0.f, ss = 0.f;
-    if (KIND == 2) {
+    if (KIND >= 2) {
       if (c == 0 && onv) {
         for (int g = 0; g < NS; ++g) o += po[g][x];
-        o = fmaf(skip, cv, o);
-        reinterpret_cast<float*>(out)[(size_t)t * H * V + (size_t)hd * V + x] = o * cg / (1.f + expf(-cg));
+        if (KIND == 2) o = fmaf(skip, cv, o) * cg / (1.f + expf(-cg));
+        reinterpret_cast<float*>(out)[(size_t)t * H * V + (size_t)hd * V + x] = o;
       }
       continue;      // po is next written after the next token's first barrier
     }
@@ -336,17 +363,18 @@ extern "C" long long k8s_gated_scan_workspace(int T, int nseq, int H, int D, int
   return 2 * chunks * H * ((long long)D * V + D + 2);
 }
 
-extern "C" int k8s_gated_scan(void* out, const float* proj, long ld, int kind, int cq, int ck, int cv, int ci, int cf,
+extern "C" int k8s_gated_scan(void* out, const void* proj, long ld, int kind, int cq, int ck, int cv, int ci, int cf,
                               int cg, const void* fbias, const void* ibias, const void* lower, const void* normw,
                               float* state, const int* cu_q, const int* seq_slots, const int* positions, int nseq, int H,
                               int D, int V, float eps, float cap, int f32, int T, int Lc, float* ws, const float* aux,
                               long ldaux, const float* hpar, int R, hipStream_t s) {
   if (nseq <= 0) return 0;
-  if (H <= 0 || H > 65535 || D <= 0 || D > 256 || V <= 0 || V > 256 || kind < 0 || kind > 2) return -1;
+  if (H <= 0 || H > 65535 || D <= 0 || D > 256 || V <= 0 || V > 256 || kind < 0 || kind > 3) return -1;
   if (kind == 2 && (aux == nullptr || hpar == nullptr || R <= 0 || H % R)) return -1;
+  if (kind == 3 && (hpar == nullptr || R <= 0 || H % R)) return -1;
   if (kind == 0 && lower == nullptr) return -1;
   if (kind == 1 && !(cap > 0.f)) return -1;
-  const int m = (kind == 2 || V > D) ? V : D, DX = (m + 63) / 64 * 64;
+  const int m = (kind >= 2 || V > D) ? V : D, DX = (m + 63) / 64 * 64;
   int ch = 16;
   while (ch < 64 && DX * ((D + ch - 1) / ch) > 1024) ch *= 2;
   if (DX * ((D + ch - 1) / ch) > 1024) return -2;
@@ -354,7 +382,8 @@ extern "C" int k8s_gated_scan(void* out, const float* proj, long ld, int kind, i
   const ScanCols co{cq, ck, cv, ci, cf, cg};
 #define K8S_GS(TA, CH, KIND, MODE, GX, LOC, START)                                                                  \
   gated_scan_kernel<TA, CH, KIND, MODE><<<dim3(GX, H), block, 0, s>>>(                                              \
-      (TA*)out, proj, ld, co, (const TA*)fbias, (const TA*)ibias, (const TA*)lower, (const TA*)normw, state, cu_q,  \
+      (TA*)out, (const scan_in_t<TA, KIND>*)proj, ld, co, (const TA*)fbias, (const TA*)ibias, (const TA*)lower,     \
+      (const TA*)normw, state, cu_q,                                                                                \
       seq_slots, positions, H, D, V, eps, cap, nseq, Lc, LOC, START, aux, ldaux, hpar, R)
 #define K8S_GS_C(TA, KIND, MODE, GX, LOC, START)                     \
   do {                                                               \
@@ -366,7 +395,8 @@ extern "C" int k8s_gated_scan(void* out, const float* proj, long ld, int kind, i
   do {                                                           \
     if (kind == 0) K8S_GS_C(TA, 0, MODE, GX, LOC, START);        \
     else if (kind == 1) K8S_GS_C(TA, 1, MODE, GX, LOC, START);   \
-    else K8S_GS_C(float, 2, MODE, GX, LOC, START);               \
+    else if (kind == 2) K8S_GS_C(float, 2, MODE, GX, LOC, START); \
+    else K8S_GS_C(TA, 3, MODE, GX, LOC, START);                  \
   } while (0)
 #define K8S_GS_T(MODE, GX, LOC, START)                      \
   do {                                                      \
@@ -385,7 +415,7 @@ extern "C" int k8s_gated_scan(void* out, const float* proj, long ld, int kind, i
   int pz = (D * V + D + 1023) / 1024;
   pz = pz < 1 ? 1 : (pz > 64 ? 64 : pz);
   const dim3 pgrid(nseq, H, pz);
-  if (kind != 1)     // one decay per key channel (KIND 2: the head's, repeated)
+  if (kind != 1)     // one decay per key channel (KIND 2, 3: the head's, repeated)
     gated_prefix_kernel<0><<<pgrid, 256, 0, s>>>(start, loc, state, cu_q, seq_slots, positions, H, D, V, Lc);
   else
     gated_prefix_kernel<1><<<pgrid, 256, 0, s>>>(start, loc, state, cu_q, seq_slots, positions, H, D, V, Lc);

@@ -271,13 +271,19 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(TA* __restrict__ c
 // of KB <= 64 cached rows staged in LDS as fp32 and shared by the heads; lane l scores key l of the block
 // ((q_abs . c + q_rot . k_rot) * scale), the block joins a running softmax, and lane l accumulates latent
 // dimensions l, l + 64, ... of sum_j p_j c_j.  out [T, H, C] = that sum / the softmax denominator.  `sinks` [H] fp32
-// (optional): the denominator of head h holds one more term e^sinks[h], which has no key and no value.
+// (optional): the denominator of head h holds one more term e^sinks[h], which has no key and no value.  `gate` (optional,
+// row stride ldg): head h's result is multiplied by sigmoid(gate[t, h]) (whatever linear map follows per head).
+template <typename TA>
+__device__ __forceinline__ float head_gate(const TA* gate, long ldg, int t, int hd) {
+  return gate != nullptr ? 1.f / (1.f + expf(-ldf(gate, (size_t)t * ldg + hd))) : 1.f;
+}
 template <typename TA, int NACC>
 __global__ void latent_attention_kernel(TA* __restrict__ out, const TA* __restrict__ q_abs, const TA* __restrict__ q,
                                         const TA* __restrict__ cache, const int* __restrict__ block_tables,
                                         int max_blocks, const int* __restrict__ tok_seq,
                                         const int* __restrict__ positions, int C, int R, int H, int Dn, int window,
-                                        float scale, int bs, int KB, const float* __restrict__ sinks) {
+                                        float scale, int bs, int KB, const float* __restrict__ sinks,
+                                        const TA* __restrict__ gate, long ldg) {
   extern __shared__ float smem[];
   const int t = blockIdx.x;
   const int p = positions[t];
@@ -343,6 +349,7 @@ __global__ void latent_attention_kernel(TA* __restrict__ out, const TA* __restri
         const float sk = sinks[hd], mx = fmaxf(m, sk), am = expf(m - mx);
         inv = am / (l * am + expf(sk - mx));
       }
+      inv *= head_gate(gate, ldg, t, hd);
 #pragma unroll
       for (int i = 0; i < NACC; ++i) {
         const int d = lane + 64 * i;
@@ -372,7 +379,8 @@ __global__ __launch_bounds__(64 * NWV) void latent_attention_mfma_kernel(
     bf16_t* __restrict__ out, float* __restrict__ pacc, float* __restrict__ pml, const bf16_t* __restrict__ q_abs,
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ cache, const int* __restrict__ block_tables, int max_blocks,
     const int* __restrict__ tok_seq, const int* __restrict__ positions, const int* __restrict__ cu_q, int C, int R,
-    int H, int Dn, int window, float scale, int bs, int nsplit, const float* __restrict__ sinks, int bt_lds) {
+    int H, int Dn, int window, float scale, int bs, int nsplit, const float* __restrict__ sinks, int bt_lds,
+    const bf16_t* __restrict__ gate, long ldg) {
   extern __shared__ __attribute__((aligned(16))) char smem_b[];
   char* klds = smem_b;               // [32][L + 8] bf16; then (bt_lds) the block-table entries of the keys this block reads
   const int hg = blockIdx.y;
@@ -581,6 +589,7 @@ __global__ __launch_bounds__(64 * NWV) void latent_attention_mfma_kernel(
         const float sk = sinks[hd], mx = fmaxf(m_i[i], sk), am = expf(m_i[i] - mx);
         inv = am / (l_i[i] * am + expf(sk - mx));
       }
+      inv *= head_gate(gate, ldg, t, hd);
 #pragma unroll
       for (int n = 0; n < NDB; ++n)
         if (n < ndb) out[((size_t)t * H + hd) * C + 16 * n + li] = f2bf(o[n][i] * inv);
@@ -601,7 +610,8 @@ __global__ __launch_bounds__(64 * NWV) void latent_attention_mfma_kernel(
 // the latent columns)
 __global__ void latent_merge_kernel(bf16_t* __restrict__ out, const float* __restrict__ pacc,
                                     const float* __restrict__ pml, const int* __restrict__ positions, int C, int H,
-                                    int HP, int nsplit, const float* __restrict__ sinks) {
+                                    int HP, int nsplit, const float* __restrict__ sinks,
+                                    const bf16_t* __restrict__ gate, long ldg) {
   const int t = blockIdx.x, hd = blockIdx.y;
   const int d0 = blockIdx.z * blockDim.x + threadIdx.x, dstep = blockDim.x * gridDim.z;
   if (positions[t] < 0) {
@@ -616,13 +626,14 @@ __global__ void latent_merge_kernel(bf16_t* __restrict__ out, const float* __res
     const float ms = pml[(rec0 + s) * 2];
     if (ms != -INFINITY) den += expf(ms - M) * pml[(rec0 + s) * 2 + 1];
   }
+  const float gh = head_gate(gate, ldg, t, hd);
   for (int d = d0; d < C; d += dstep) {
     float a = 0.f;
     for (int s = 0; s < nsplit; ++s) {
       const float ms = pml[(rec0 + s) * 2];
       if (ms != -INFINITY) a += expf(ms - M) * pacc[(rec0 + s) * C + d];
     }
-    out[((size_t)t * H + hd) * C + d] = f2bf(a / den);
+    out[((size_t)t * H + hd) * C + d] = f2bf(a / den * gh);
   }
 }
 
@@ -712,8 +723,9 @@ extern "C" int k8s_latent_kv_write(void* cache, const void* dkv, const void* nor
 extern "C" int k8s_latent_attention(void* out, const void* q_abs, const void* q, const void* cache,
                                     const int* block_tables, int max_blocks, const int* tok_seq, const int* positions,
                                     int T, int C, int R, int H, int Dn, int window, float scale, int bs, int f32,
-                                    const float* sinks, hipStream_t s) {
+                                    const float* sinks, const void* gate, long ldg, hipStream_t s) {
   if (T <= 0) return 0;
+  if (gate != nullptr && ldg < H) return -1;
   if (C <= 0 || C > 512 || R < 0 || H <= 0 || bs <= 0) return -1;
   const int L = C + R;
   const int nw = H < 8 ? H : 8;
@@ -726,7 +738,7 @@ extern "C" int k8s_latent_attention(void* out, const void* q_abs, const void* q,
 #define K8S_LA(TA, NA) \
   latent_attention_kernel<TA, NA><<<T, nw * 64, lds, s>>>((TA*)out, (const TA*)q_abs, (const TA*)q, (const TA*)cache, \
                                                           block_tables, max_blocks, tok_seq, positions, C, R, H, Dn, \
-                                                          window, scale, bs, KB, sinks)
+                                                          window, scale, bs, KB, sinks, (const TA*)gate, ldg)
 #define K8S_LA_T(TA)                  \
   do {                                \
     if (nacc <= 1) K8S_LA(TA, 1);     \
@@ -753,8 +765,10 @@ extern "C" int k8s_latent_attention_mfma(void* out, float* pacc, float* pml, con
                                          const void* cache, const int* block_tables, int max_blocks,
                                          const int* tok_seq, const int* positions, int T, int C, int R, int H, int Dn,
                                          int window, float scale, int bs, int nsplit, const int* cu_q, int nseq,
-                                         int max_qlen, const float* sinks, hipStream_t s) {
+                                         int max_qlen, const float* sinks, const void* gate, long ldg,
+                                         hipStream_t s) {
   if (T <= 0) return 0;
+  if (gate != nullptr && ldg < H) return -1;
   if (!k8s_latent_mfma_ok(C, R, Dn) || H <= 0 || bs <= 0 || nsplit < 1 || (nsplit > 1 && (!pacc || !pml))) return -1;
   const int L = C + R, HG = (H + 15) / 16;
   const size_t lds = (size_t)32 * (L + 8) * 2;
@@ -769,11 +783,13 @@ extern "C" int k8s_latent_attention_mfma(void* out, float* pacc, float* pml, con
     if (tiles)                                                                                                        \
       latent_attention_mfma_kernel<NDB, NKK, 4, EX><<<grid, 256, lds + bt_bytes, s>>>(                                             \
           (bf16_t*)out, pacc, pml, (const bf16_t*)q_abs, (const bf16_t*)q, (const bf16_t*)cache, block_tables,        \
-          max_blocks, tok_seq, positions, cu_q, C, R, H, Dn, window, scale, bs, nsplit, sinks, bt_lds);               \
+          max_blocks, tok_seq, positions, cu_q, C, R, H, Dn, window, scale, bs, nsplit, sinks, bt_lds,                \
+          (const bf16_t*)gate, ldg);                                                                                   \
     else                                                                                                              \
       latent_attention_mfma_kernel<NDB, NKK, 1, EX><<<grid, 64, lds, s>>>(                                             \
           (bf16_t*)out, pacc, pml, (const bf16_t*)q_abs, (const bf16_t*)q, (const bf16_t*)cache, block_tables,        \
-          max_blocks, tok_seq, positions, cu_q, C, R, H, Dn, window, scale, bs, nsplit, sinks, 0);                    \
+          max_blocks, tok_seq, positions, cu_q, C, R, H, Dn, window, scale, bs, nsplit, sinks, 0,                     \
+          (const bf16_t*)gate, ldg);                                                                                   \
   } while (0)
   if (C == 512 && L == 576) K8S_LM(32, 18, true);        // sizes that fill an instantiation exactly
   else if (C == 256 && L == 320) K8S_LM(16, 10, true);
@@ -787,6 +803,6 @@ extern "C" int k8s_latent_attention_mfma(void* out, float* pacc, float* pml, con
 #undef K8S_LM
   if (nsplit > 1)
     latent_merge_kernel<<<dim3(T, H, (C + 127) / 128), 128, 0, s>>>((bf16_t*)out, pacc, pml, positions, C, H, HG * 16,
-                                                                    nsplit, sinks);
+                                                                    nsplit, sinks, (const bf16_t*)gate, ldg);
   return (int)hipGetLastError();
 }

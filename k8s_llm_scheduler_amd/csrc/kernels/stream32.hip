@@ -89,6 +89,52 @@ __global__ __launch_bounds__(256) void postnorm_kernel(float* __restrict__ x, co
   }
 }
 
+// Norm of a sublayer's output ahead of the sum: x[t] += branch[t] / sqrt(mean(branch[t]^2) + eps) * w, in fp32; `out`
+// (optional) receives the new row in the activation type, for the sublayer that reads the stream next.  One workgroup
+// per row; NR > 0: the row's branch values stay in registers between the two passes (W <= 256 NR), else they are read
+// again.
+template <typename TB, typename TA, int NR>
+__global__ __launch_bounds__(256) void branchnorm_kernel(float* __restrict__ x, const TB* __restrict__ branch,
+                                                         const TA* __restrict__ w, float eps, TA* __restrict__ out,
+                                                         int W) {
+  __shared__ float red[16];
+  const size_t base = (size_t)blockIdx.x * W;
+  float ss = 0.f;
+  if constexpr (NR > 0) {
+    float v[NR], xv[NR];
+#pragma unroll
+    for (int n = 0; n < NR; ++n) {
+      const int i = threadIdx.x + 256 * n;
+      v[n] = i < W ? ldf(branch, base + i) : 0.f;
+      xv[n] = i < W ? x[base + i] : 0.f;
+    }
+#pragma unroll
+    for (int n = 0; n < NR; ++n) ss += v[n] * v[n];
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+    for (int n = 0; n < NR; ++n) {
+      const int i = threadIdx.x + 256 * n;
+      if (i >= W) continue;
+      const float y = fmaf(v[n] * inv, ldf(w, i), xv[n]);
+      x[base + i] = y;
+      if (out != nullptr) stf(out, base + i, y);
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += blockDim.x) {
+      const float v = ldf(branch, base + i);
+      ss += v * v;
+    }
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+    for (int i = threadIdx.x; i < W; i += blockDim.x) {
+      const float y = fmaf(ldf(branch, base + i) * inv, ldf(w, i), x[base + i]);
+      x[base + i] = y;
+      if (out != nullptr) stf(out, base + i, y);
+    }
+  }
+}
+
 // out[t, c] = y[t, c] * f(gate[t, c]) with f = sigmoid (kind 0) or silu (kind 1); y and gate are row-strided views.
 template <typename TY, typename TA>
 __global__ void gate_mul_kernel(TA* __restrict__ out, const TY* __restrict__ y, long ldy, const TA* __restrict__ gate,
@@ -104,7 +150,7 @@ __global__ void gate_mul_kernel(TA* __restrict__ out, const TY* __restrict__ y, 
 
 // kinds: 0 gelu_tanh(g) * u, 1 g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, +-limit)
 // (limit <= 0: no clamp), 5 relu(g) * u -- these read [T, 2F] = [gate | up]; 2 tanh, 3 silu, 4 erf-gelu,
-// 6 limit * tanh(x / limit): elementwise on [T, F].
+// 6 limit * tanh(x / limit), 7 relu(x)^2: elementwise on [T, F].
 // Elementwise kinds take a factor per row: logical row i is row row_map[i] (or i) and its input is multiplied by
 // row_scale[i] before the function (experts whose router weight scales their input).
 template <typename TA>
@@ -122,6 +168,7 @@ __global__ void act_kernel(TA* __restrict__ out, const TA* __restrict__ x, int T
       y = kind == 2   ? tanhf(v)
           : kind == 3 ? v / (1.f + expf(-v))
           : kind == 4 ? 0.5f * v * (1.f + erff(v * 0.7071067811865476f))
+          : kind == 7 ? (v > 0.f ? v * v : 0.f)
                       : limit * tanhf(v / limit);
     } else {
       float g = ldf(x, t * 2 * F + c), u = ldf(x, t * 2 * F + F + c);
@@ -144,12 +191,18 @@ __global__ void act_kernel(TA* __restrict__ out, const TA* __restrict__ x, int T
 // out[t] = ca * a[t] / rms(a[t]) * wa + cb * b[t] / rms(b[t]) * wb (b optional): the outputs of two mixers that run side
 // by side, each normed over the row in fp32, joined.  One workgroup per row.  `lda`: the row stride of a (a view into a
 // wider projection).  groups > 1 (a alone): every one of that many equal consecutive parts of the row is divided by its
-// own root mean square, one wave per part.
+// own root mean square, one wave per part.  `gate` (optional, output type, row stride ldg): every element of the result
+// times sigmoid(gate) (gkind 0) or silu(gate) (gkind 1).
+template <typename TO>
+__device__ __forceinline__ float gate_of(const TO* gate, size_t i, int gkind) {
+  const float g = ldf(gate, i), s = 1.f / (1.f + expf(-g));
+  return gkind == 1 ? g * s : s;
+}
 template <typename TA, typename TO>
 __global__ __launch_bounds__(256) void norm_mix_kernel(TO* __restrict__ out, const TA* __restrict__ a, long lda,
                                                        const TA* __restrict__ wa, const TA* __restrict__ b,
                                                        const TA* __restrict__ wb, float eps, float ca, float cb, int W,
-                                                       int groups) {
+                                                       int groups, const TO* __restrict__ gate, long ldg, int gkind) {
   __shared__ float red[16];
   const size_t base = (size_t)blockIdx.x * W;
   const TA* ar = a + (size_t)blockIdx.x * lda;
@@ -164,7 +217,10 @@ __global__ __launch_bounds__(256) void norm_mix_kernel(TO* __restrict__ out, con
       }
       sg = wave_sum(sg);
       const float inv = ca / sqrtf(sg / (float)Wg + eps);
-      for (int i = lane; i < Wg; i += 64) stf(out, base + o + i, ldf(ar, o + i) * inv * ldf(wa, o + i));
+      for (int i = lane; i < Wg; i += 64) {
+        const float y = ldf(ar, o + i) * inv * ldf(wa, o + i);
+        stf(out, base + o + i, gate != nullptr ? y * gate_of(gate, (size_t)blockIdx.x * ldg + o + i, gkind) : y);
+      }
     }
     return;
   }
@@ -187,6 +243,7 @@ __global__ __launch_bounds__(256) void norm_mix_kernel(TO* __restrict__ out, con
   for (int i = threadIdx.x; i < W; i += blockDim.x) {
     float y = ldf(ar, i) * ia * ldf(wa, i);
     if (b != nullptr) y += ldf(b, base + i) * ib * ldf(wb, i);
+    if (gate != nullptr) y *= gate_of(gate, (size_t)blockIdx.x * ldg + i, gkind);
     stf(out, base + i, y);
   }
 }
@@ -391,14 +448,15 @@ extern "C" int k8s_resnorm(float* x, const void* branch, const void* branch2, fl
 }
 
 extern "C" int k8s_norm_mix(void* out, const void* a, long lda, const void* wa, const void* b, const void* wb,
-                            float eps, float ca, float cb, int T, int W, int groups, int in_f32, int out_f32,
-                            hipStream_t s) {
+                            float eps, float ca, float cb, int T, int W, int groups, const void* gate, long ldg,
+                            int gkind, int in_f32, int out_f32, hipStream_t s) {
   if (T <= 0) return 0;
   if (W <= 0 || a == nullptr || wa == nullptr || (b != nullptr && wb == nullptr) || lda < W) return -1;
   if (groups < 1 || W % groups || (groups > 1 && b != nullptr)) return -1;
+  if (gate != nullptr && (ldg < W || gkind < 0 || gkind > 1)) return -1;
 #define K8S_NM(TA, TO)                                                                                             \
   norm_mix_kernel<TA, TO><<<T, 256, 0, s>>>((TO*)out, (const TA*)a, lda, (const TA*)wa, (const TA*)b, (const TA*)wb, \
-                                            eps, ca, cb, W, groups)
+                                            eps, ca, cb, W, groups, (const TO*)gate, ldg, gkind)
   if (in_f32 && out_f32) K8S_NM(float, float);
   else if (in_f32) K8S_NM(float, bf16_t);
   else if (out_f32) K8S_NM(bf16_t, float);
@@ -417,6 +475,28 @@ extern "C" int k8s_postnorm(float* x, const void* branch, const void* branch2, f
   else
     postnorm_kernel<bf16_t><<<T, 256, 0, s>>>(x, (const bf16_t*)branch, (const bf16_t*)branch2, alpha, c1, c2, gain,
                                               eps, (bf16_t*)out, W);
+  return (int)hipGetLastError();
+}
+
+// branch_f32: the branch is fp32 whatever the activation type of w and out
+extern "C" int k8s_branchnorm(float* x, const void* branch, const void* w, float eps, void* out, int T, int W,
+                              int branch_f32, int f32, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (W <= 0 || x == nullptr || branch == nullptr || w == nullptr || (f32 && !branch_f32)) return -1;
+#define K8S_BN(TB, TA, NR) \
+  branchnorm_kernel<TB, TA, NR><<<T, 256, 0, s>>>(x, (const TB*)branch, (const TA*)w, eps, (TA*)out, W)
+#define K8S_BN_T(TB, TA)                       \
+  do {                                         \
+    if (W <= 512) K8S_BN(TB, TA, 2);           \
+    else if (W <= 2048) K8S_BN(TB, TA, 8);     \
+    else if (W <= 4096) K8S_BN(TB, TA, 16);    \
+    else K8S_BN(TB, TA, 0);                    \
+  } while (0)
+  if (f32) K8S_BN_T(float, float);
+  else if (branch_f32) K8S_BN_T(float, bf16_t);
+  else K8S_BN_T(bf16_t, bf16_t);
+#undef K8S_BN_T
+#undef K8S_BN
   return (int)hipGetLastError();
 }
 
@@ -443,7 +523,7 @@ extern "C" int k8s_act(void* out, const void* x, int T, int F, int kind, float l
                        const float* row_scale, const int* row_map, int f32, hipStream_t s) {
   if (T <= 0 || F <= 0) return 0;
   const bool gated = kind < 2 || kind == 5;
-  if (kind < 0 || kind > 6 || (gated && (row_scale != nullptr || row_map != nullptr)) || (kind == 6 && !(limit > 0.f)))
+  if (kind < 0 || kind > 7 || (gated && (row_scale != nullptr || row_map != nullptr)) || (kind == 6 && !(limit > 0.f)))
     return -1;
   const size_t n = (size_t)T * F;
   const int blocks = (int)((n + 255) / 256 > 4096 ? 4096 : (n + 255) / 256);

@@ -15,10 +15,10 @@ def _architecture(c: dict) -> str:
 
 def load_config(name_or_path: str):
     """The configuration object of a preset or checkpoint."""
-    from . import nukizen, putulorn, rupatar, semanex
+    from . import katidra, nukizen, putulorn, rupatar, semanex
     from .config import get_config
 
-    designs = (putulorn, rupatar, nukizen, semanex)
+    designs = (putulorn, rupatar, nukizen, semanex, katidra)
     for d in designs:
         if name_or_path in d.PRESETS:
             return d.PRESETS[name_or_path]
@@ -36,6 +36,7 @@ def load_config(name_or_path: str):
 def model_class(cfg):
     """The model class of a configuration object."""
     from .config import LlamaConfig
+    from .katidra import KatidraConfig, KatidraModel
     from .llama import LlamaModel
     from .nukizen import NukizenConfig, NukizenModel
     from .putulorn import PutulornConfig, PutulornModel
@@ -50,6 +51,8 @@ def model_class(cfg):
         return NukizenModel
     if isinstance(cfg, SemanexConfig):
         return SemanexModel
+    if isinstance(cfg, KatidraConfig):
+        return KatidraModel
     if isinstance(cfg, LlamaConfig):
         return LlamaModel
     raise TypeError(f"no model class for {type(cfg).__name__}")

@@ -38,7 +38,7 @@ from ..ops import reference as ref
 from ..ops import seqmix as sm
 from ..parallel import TPGroup
 from . import stream
-from .stream import StreamModel
+from .stream import StreamModel, stack_rows
 
 ARCHITECTURE = "Semanex"
 MIXERS = ("latent_attention", "parallel")
@@ -335,20 +335,6 @@ class _Layer:
     w_down: Optional[torch.Tensor] = None
 
 
-def _stack(parts, align: int = 16):
-    """Rows of several projections of one input, every part padded to a multiple of ``align`` rows (16-byte aligned
-    column offsets in the product): (weight, column offset of every part)."""
-    rows, cols, at = [], {}, 0
-    for key, w in parts:
-        cols[key] = at
-        rows.append(w)
-        pad = (-w.shape[0]) % align
-        if pad:
-            rows.append(torch.zeros(pad, w.shape[1], dtype=w.dtype))
-        at += w.shape[0] + pad
-    return torch.cat(rows), cols
-
-
 class SemanexModel(StreamModel):
     def __init__(self, cfg: SemanexConfig, tp: Optional[TPGroup] = None, device="cpu", dtype=torch.bfloat16,
                  seed: int = 0, weights: Optional[str] = None, tensors: Optional[Dict[str, torch.Tensor]] = None,
@@ -383,7 +369,7 @@ class SemanexModel(StreamModel):
         H, Dn, R, V, C = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
         if m.rot_dims % 2 or not 0 < m.rot_dims <= R:
             raise ValueError(f"{where}: rot.dims {m.rot_dims} must be even, positive and at most rot_dim {R}")
-        w_in, cols = _stack((("dq", get(p + "dq").cpu()), ("dkv", get(p + "dkv").cpu()), ("g", get(p + "g").cpu())))
+        w_in, cols = stack_rows((("dq", get(p + "dq").cpu()), ("dkv", get(p + "dkv").cpu()), ("g", get(p + "g").cpu())))
         return _Latent(m, t(w_in), cols, t(get(p + "dq.norm")), t(get(p + "uq")), t(get(p + "dkv.norm")),
                        t(get(p + "uk").view(H, Dn, C).transpose(1, 2)), t(get(p + "uv").view(H, V, C)),
                        self._f(get(p + "sink")), t(get(p + "o")), self._rope_table(m.rot_dims, m.rot_base))
@@ -398,7 +384,7 @@ class SemanexModel(StreamModel):
         if max(r.state, r.vdim) > sm.gated_scan_max_dim():
             raise ValueError(f"{where}: state {r.state} x {r.vdim} exceeds the kernels' {sm.gated_scan_max_dim()}")
         q = p + "left."
-        w_in, cols = _stack(tuple((s, get(q + s).cpu()) for s in ("q", "k", "v", "g")))
+        w_in, cols = stack_rows(tuple((s, get(q + s).cpu()) for s in ("q", "k", "v", "g")))
         left = _Capped(a, t(w_in), cols, t(get(q + "q.norm")), t(get(q + "k.norm")), t(get(q + "o")))
         q = p + "right."
         r.conv = int(get(q + "conv").shape[1])                 # the taps are what the checkpoint holds

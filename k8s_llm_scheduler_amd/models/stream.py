@@ -26,6 +26,20 @@ def save_checkpoint(config_json: dict, tensors: Dict[str, torch.Tensor], path: P
     (path / "config.json").write_text(json.dumps(config_json))
 
 
+def stack_rows(parts, align: int = 16):
+    """Rows of several projections of one input, every part padded to a multiple of ``align`` rows (16-byte aligned
+    column offsets in the product): (weight, column offset of every part)."""
+    rows, cols, at = [], {}, 0
+    for key, w in parts:
+        cols[key] = at
+        rows.append(w)
+        pad = (-w.shape[0]) % align
+        if pad:
+            rows.append(torch.zeros(pad, w.shape[1], dtype=w.dtype))
+        at += w.shape[0] + pad
+    return torch.cat(rows), cols
+
+
 class StreamModel:
     stateful = True          # per-slot recurrent state: the engine passes each sequence's slot, keeps prefix caching,
     prefill_graphs = False   # speculative decoding and padded prefill graphs off

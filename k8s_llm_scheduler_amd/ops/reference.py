@@ -498,6 +498,7 @@ def write_token_stop(s: int, tok: int, tokens, ctx_inc, hist, steps, stop) -> No
 
 # ----------------------------------------------------------------------------- fp32 residual stream, gated activations
 ACT_GELU_TANH, ACT_SWISH_CLAMP, ACT_TANH, ACT_SILU, ACT_GELU_ERF, ACT_RELU, ACT_SOFTCAP = 0, 1, 2, 3, 4, 5, 6
+ACT_RELU2 = 7
 
 
 def embed_rows(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
@@ -535,6 +536,13 @@ def postnorm(x: torch.Tensor, branch, branch2, alpha: float, c1: float, c2: floa
     return x.to(out_dtype) if out_dtype is not None else None
 
 
+def branchnorm(x: torch.Tensor, branch, w, eps: float, out_dtype):
+    """x (fp32, in place) += branch / sqrt(mean(branch^2) + eps) * w; returns the new rows in ``out_dtype`` (None: nothing)."""
+    b = branch.float()
+    x.add_(b * torch.rsqrt(b.pow(2).mean(-1, keepdim=True) + eps) * w.float())
+    return x.to(out_dtype) if out_dtype is not None else None
+
+
 GATE_SIGMOID, GATE_SILU = 0, 1
 
 
@@ -549,17 +557,19 @@ def gate_mul(y: torch.Tensor, gate: torch.Tensor, kind: int) -> torch.Tensor:
 
 def act(x: torch.Tensor, kind: int, limit: float = 0.0, alpha: float = 1.0, row_scale=None, row_map=None) -> torch.Tensor:
     """Gated kinds (ACT_GELU_TANH, ACT_SWISH_CLAMP, ACT_RELU: relu(g) u) take [T, 2F] = [gate | up] and return [T, F];
-    ACT_TANH / ACT_SILU / ACT_GELU_ERF / ACT_SOFTCAP (limit tanh(x / limit)) are elementwise and take a factor per row:
+    ACT_TANH / ACT_SILU / ACT_GELU_ERF / ACT_RELU2 (relu squared) / ACT_SOFTCAP (limit tanh(x / limit)) are elementwise and take a factor per row:
     logical row i is row ``row_map[i]`` (or i), its input times ``row_scale[i]``."""
     if kind == ACT_SOFTCAP:
         return (limit * torch.tanh(x.float() / limit)).to(x.dtype)
-    if kind in (ACT_TANH, ACT_SILU, ACT_GELU_ERF):
+    if kind in (ACT_TANH, ACT_SILU, ACT_GELU_ERF, ACT_RELU2):
         f = x.float()
         if row_scale is not None:
             sc = row_scale.float()
             if row_map is not None:
                 sc = torch.zeros(x.shape[0]).index_copy_(0, row_map.long(), sc)
             f = f * sc.unsqueeze(-1)
+        if kind == ACT_RELU2:
+            return torch.relu(f).square().to(x.dtype)
         if kind == ACT_GELU_ERF:
             return (0.5 * f * (1.0 + torch.erf(f / math.sqrt(2.0)))).to(x.dtype)
         return (torch.tanh(f) if kind == ACT_TANH else f * torch.sigmoid(f)).to(x.dtype)
@@ -680,10 +690,10 @@ def latent_kv_write(cache, dkv, normw, q, cos_sin, positions, slot_mapping, C: i
 
 
 def latent_attention(q_abs, q, cache, block_tables, tok_seq, positions, C: int, R: int, H: int, Dn: int,
-                     window: int, scale: float, block_size: int, out_dtype, sinks=None):
+                     window: int, scale: float, block_size: int, out_dtype, sinks=None, gate=None):
     """Token t of sequence tok_seq[t] at position p attends the cached rows of positions max(0, p - window + 1) .. p
     (window <= 0: all): score = (q_abs . c + q_rot . k_rot) * scale, softmax (``sinks`` [H]: one more term e^sinks[h]
-    in head h's denominator), returns sum p c  [T, H, C]."""
+    in head h's denominator), returns sum p c  [T, H, C]; ``gate`` [T, H]: times sigmoid(gate) per head."""
     T = q_abs.shape[0]
     out = torch.zeros(T, H, C)
     qa = q_abs.float().view(T, H, C)
@@ -703,6 +713,8 @@ def latent_attention(q_abs, q, cache, block_tables, tok_seq, positions, C: int, 
             out[t] = (e / (e.sum(-1, keepdim=True) + torch.exp(sinks.float().view(H, 1) - mx))) @ rows[:, :C]
             continue
         out[t] = torch.softmax(s, -1) @ rows[:, :C]
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float()).unsqueeze(-1)
     return out.to(out_dtype)
 
 
@@ -875,7 +887,7 @@ def window_attention(q, gate, kcache, vcache, kpool, vpool, block_tables, tok_se
 
 
 # ----------------------------------------------------------------------------- gated matrix-state recurrences
-SCAN_HGRN2, SCAN_MLSTM, SCAN_SSD = 0, 1, 2
+SCAN_HGRN2, SCAN_MLSTM, SCAN_SSD, SCAN_DECAY = 0, 1, 2, 3
 
 
 def gated_scan_record(kind: int, D: int, V: int) -> int:
@@ -911,6 +923,30 @@ def ssd_scan(proj, cols: dict, aux, head_params, state, cu_q, seq_slots, positio
     return out.reshape(T, H * V) * gate * torch.sigmoid(gate)
 
 
+def decay_scan(proj, cols: dict, decay, state, cu_q, seq_slots, positions, H: int, G: int, D: int, V: int):
+    """Linear attention under a constant decay per head: q, k (G D each) and v (H V) of ``proj`` at the columns ``cols``
+    pass silu; S <- decay[h] S + k v^T, y = S^T q with the q, k of group h // (H / G).  fp32 [T, H V]; ``state``
+    [slots, H, D V] fp32."""
+    T = proj.shape[0]
+    silu = torch.nn.functional.silu
+    part = lambda key, n, d: silu(proj[:, cols[key]:cols[key] + n * d].float()).view(T, n, d)
+    q, k = (part(key, G, D).repeat_interleave(H // G, 1) for key in ("q", "k"))
+    v = part("v", H, V)
+    out = torch.zeros(T, H, V)
+    cu = cu_q.tolist()
+    for s in range(len(cu) - 1):
+        a, b = cu[s], cu[s + 1]
+        if b <= a or int(positions[a]) < 0:
+            continue
+        slot = int(seq_slots[s])
+        S = torch.zeros(H, D, V) if int(positions[a]) == 0 else state[slot].view(H, D, V).clone()
+        for t in range(a, b):
+            S = decay.float().view(H, 1, 1) * S + k[t].unsqueeze(2) * v[t].unsqueeze(1)
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S.reshape(H, D * V)
+    return out.reshape(T, H * V)
+
+
 def gated_scan(proj, kind: int, cols: dict, fbias, ibias, lower, normw, state, cu_q, seq_slots, positions, H: int,
                D: int, V: int, eps: float, cap: float, out_dtype, aux=None, head_params=None, groups: int = 0):
     """``proj`` fp32 [T, ld] holds the parts at the column offsets ``cols``; ``state`` [slots, H, record] fp32.
@@ -920,6 +956,8 @@ def gated_scan(proj, kind: int, cols: dict, fbias, ibias, lower, normw, state, c
     with q = zq / sqrt(D), y = o / rms(o) * normw [H V] * sigmoid(zg).  A portion at position 0 starts from zero."""
     if kind == SCAN_SSD:
         return ssd_scan(proj, cols, aux, head_params, state, cu_q, seq_slots, positions, H, groups, D, V)
+    if kind == SCAN_DECAY:
+        return decay_scan(proj, cols, head_params, state, cu_q, seq_slots, positions, H, groups, D, V)
     T = proj.shape[0]
     pf = proj.float()
     out = torch.zeros(T, H, V)
@@ -1093,16 +1131,22 @@ def rglru_scan(u, gates, gate_bias, decay_rate, proj, ycol: int, ybias, state, c
     return (out * y).to(out_dtype)
 
 
-def norm_mix(a, wa, b, wb, eps: float, ca: float, cb: float, out_dtype, groups: int = 1):
+def norm_mix(a, wa, b, wb, eps: float, ca: float, cb: float, out_dtype, groups: int = 1, gate=None,
+             gate_kind: int = GATE_SIGMOID):
     """ca * a / rms(a) * wa + cb * b / rms(b) * wb  (rows; ``b`` may be None); ``groups`` > 1: the root mean square of
-    each of that many equal consecutive parts of a row by itself."""
+    each of that many equal consecutive parts of a row by itself; ``gate``: the result times sigmoid(gate) / silu(gate)."""
     af = a.float()
+    g = 1.0
+    if gate is not None:
+        g = torch.sigmoid(gate.float())
+        if gate_kind == GATE_SILU:
+            g = g * gate.float()
     if groups > 1:
         ag = af.reshape(af.shape[0], groups, -1)
         y = ca * (ag * torch.rsqrt(ag.pow(2).mean(-1, keepdim=True) + eps)).reshape(af.shape) * wa.float()
-        return y.to(out_dtype)
+        return (y * g).to(out_dtype)
     y = ca * af * torch.rsqrt(af.pow(2).mean(-1, keepdim=True) + eps) * wa.float()
     if b is not None:
         bf = b.float()
         y = y + cb * bf * torch.rsqrt(bf.pow(2).mean(-1, keepdim=True) + eps) * wb.float()
-    return y.to(out_dtype)
+    return (y * g).to(out_dtype)

@@ -15,10 +15,11 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .reference import ACT_GELU_ERF, ACT_GELU_TANH, ACT_RELU, ACT_SILU, ACT_SOFTCAP, ACT_SWISH_CLAMP, ACT_TANH  # noqa: F401
+from .reference import ACT_GELU_ERF, ACT_GELU_TANH, ACT_RELU, ACT_RELU2, ACT_SILU, ACT_SOFTCAP, ACT_SWISH_CLAMP  # noqa: F401
+from .reference import ACT_TANH  # noqa: F401
 from .reference import CONV_NONE, CONV_SILU  # noqa: F401
 from .reference import GATE_SIGMOID, GATE_SILU  # noqa: F401
-from .reference import SCAN_HGRN2, SCAN_MLSTM, SCAN_SSD  # noqa: F401
+from .reference import SCAN_DECAY, SCAN_HGRN2, SCAN_MLSTM, SCAN_SSD  # noqa: F401
 
 BF16, F32, I32 = torch.bfloat16, torch.float32, torch.int32
 GROUP_BM = 64   # row-tile height of the grouped GEMM (gemm_any_kernel's BM)
@@ -94,24 +95,49 @@ def resnorm(x: torch.Tensor, w: Optional[torch.Tensor], eps: float, *, branch: O
 
 
 def norm_mix(a: torch.Tensor, wa: torch.Tensor, b: Optional[torch.Tensor], wb: Optional[torch.Tensor], eps: float,
-             ca: float = 1.0, cb: float = 1.0, out_dtype=None, groups: int = 1) -> torch.Tensor:
+             ca: float = 1.0, cb: float = 1.0, out_dtype=None, groups: int = 1, gate: Optional[torch.Tensor] = None,
+             gate_kind: int = GATE_SIGMOID) -> torch.Tensor:
     """ca * rms-norm(a) * wa + cb * rms-norm(b) * wb over rows [T, W] (norms in fp32; ``b`` None: the first term
     only): the outputs of two mixers that run side by side, each normed, joined.  ``a`` may be a column slice of a
     wider tensor (row stride free).  ``groups`` > 1 (``a`` alone): every one of that many equal consecutive parts of a
-    row is divided by its own root mean square."""
+    row is divided by its own root mean square.  ``gate`` [T, W] of the output type (row stride free): the result times
+    sigmoid(gate) or silu(gate), element by element."""
     out_dtype = out_dtype or a.dtype
     T, W = a.shape
+    if gate is not None and (gate.shape != a.shape or gate.dtype != out_dtype or gate.stride(1) != 1):
+        raise ValueError("norm_mix: the gate must be [T, W] of the output type with contiguous rows")
     if groups < 1 or W % groups or (groups > 1 and b is not None):
         raise ValueError(f"norm_mix: {groups} groups must divide the width {W} and go with one input")
-    if not _gpu(a, wa, b, wb):
-        return ref.norm_mix(a, wa, b, wb, eps, ca, cb, out_dtype, groups)
+    if not _gpu(a, wa, b, wb, gate):
+        return ref.norm_mix(a, wa, b, wb, eps, ca, cb, out_dtype, groups, gate, gate_kind)
     if a.stride(1) != 1:
         raise ValueError("norm_mix: rows must be contiguous")
     if b is not None and (b.shape != a.shape or b.dtype != a.dtype or wb is None):
         raise ValueError("norm_mix: the two inputs must agree in shape and dtype")
     out = torch.empty(T, W, dtype=out_dtype, device=a.device)
     _native().norm_mix(out.data_ptr(), a.data_ptr(), a.stride(0), _p(wa, a.dtype, "wa"), _p(b), _p(wb, a.dtype, "wb"),
-                       float(eps), float(ca), float(cb), T, W, int(groups), _f32(a.dtype), _f32(out_dtype), -1)
+                       float(eps), float(ca), float(cb), T, W, int(groups), gate.data_ptr() if gate is not None else 0,
+                       gate.stride(0) if gate is not None else 0, int(gate_kind), _f32(a.dtype), _f32(out_dtype), -1)
+    return out
+
+
+def branchnorm(x: torch.Tensor, branch: torch.Tensor, w: torch.Tensor, eps: float, *,
+               out_dtype=None) -> Optional[torch.Tensor]:
+    """Norm of the sublayer's output only: ``x`` (fp32 [T, W], updated in place) += rms-norm(branch) * w.  ``branch`` is
+    of w's type, or fp32.  With ``out_dtype`` (w's type) the new rows are also returned in that type: the sublayers of
+    such a design read the stream itself."""
+    if x.dtype != F32 or not x.is_contiguous():
+        raise TypeError("the residual stream is contiguous fp32")
+    if branch.shape != x.shape or branch.dtype not in (w.dtype, F32) or w.numel() != x.shape[1]:
+        raise TypeError("branchnorm: branch [T, W] of the weight's type or fp32, w [W]")
+    if out_dtype is not None and out_dtype != w.dtype:
+        raise TypeError("branchnorm: the returned rows take the weight's type")
+    if not _gpu(x, branch, w):
+        return ref.branchnorm(x, branch, w, eps, out_dtype)
+    T, W = x.shape
+    out = torch.empty(T, W, dtype=out_dtype, device=x.device) if out_dtype is not None else None
+    _native().branchnorm(_p(x), _p(branch), _p(w), float(eps), _p(out), T, W, int(branch.dtype == F32), _f32(w.dtype),
+                         -1)
     return out
 
 
@@ -159,7 +185,7 @@ def gate_mul(y: torch.Tensor, gate: torch.Tensor, kind: int = GATE_SIGMOID) -> t
 def act(x: torch.Tensor, kind: int, limit: float = 0.0, alpha: float = 1.0, *,
         row_scale: Optional[torch.Tensor] = None, row_map: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Gated kinds (ACT_GELU_TANH, ACT_SWISH_CLAMP, ACT_RELU = relu(g) u): [T, 2F] = [gate | up] -> [T, F]; ACT_TANH /
-    ACT_SILU / ACT_GELU_ERF (exact gelu) / ACT_SOFTCAP (limit tanh(x / limit)): elementwise.  Elementwise kinds take an
+    ACT_SILU / ACT_GELU_ERF (exact gelu) / ACT_RELU2 (the square of relu) / ACT_SOFTCAP (limit tanh(x / limit)): elementwise.  Elementwise kinds take an
     fp32 factor per row, ``row_scale`` [T]: logical row i is row ``row_map[i]`` (a permutation; default i) and its
     input is multiplied by ``row_scale[i]`` before the function."""
     gated = kind in (ACT_GELU_TANH, ACT_SWISH_CLAMP, ACT_RELU)
@@ -364,18 +390,23 @@ def latent_splits(T: int, H: int, max_keys: int) -> int:
 def latent_attention(q_abs: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor,
                      tok_seq: torch.Tensor, positions: torch.Tensor, C: int, R: int, H: int, Dn: int, window: int,
                      scale: float, block_size: int, max_keys: int = 0, cu_q: Optional[torch.Tensor] = None,
-                     max_qlen: int = 0, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     max_qlen: int = 0, sinks: Optional[torch.Tensor] = None,
+                     gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Sliding-window attention in the latent space over the paged cache; returns softmax-weighted latents [T, H, C].
     ``max_keys``: an upper bound of the keys any token sees (sizes the key splits; 0: the table's capacity).
     ``cu_q`` / ``max_qlen`` (the sequences' query offsets and longest portion): portions of prompts run four
     consecutive tokens per workgroup, sharing the staged cache rows.
     ``sinks`` [H] fp32: the softmax denominator of head h holds one more term e^sinks[h] (no key, no value).
+    ``gate`` [T, H] of q's type (row stride free): head h's result is multiplied by sigmoid(gate[t, h]), which commutes
+    with the value up-projection that follows.
     bf16 with 16-byte-aligned parts runs on the matrix cores; fp32 and other sizes on the plain-FMA kernel."""
     if sinks is not None and (sinks.dtype != F32 or sinks.numel() != H):
         raise ValueError("latent_attention: sinks are fp32 [H]")
-    if not _gpu(q_abs, q, cache, sinks):
+    if gate is not None and (gate.shape != (q.shape[0], H) or gate.dtype != q.dtype or gate.stride(1) != 1):
+        raise ValueError("latent_attention: the gate is [T, H] of the queries' type with contiguous rows")
+    if not _gpu(q_abs, q, cache, sinks, gate):
         return ref.latent_attention(q_abs, q, cache, block_tables, tok_seq, positions, C, R, H, Dn, window, scale,
-                                    block_size, q.dtype, sinks)
+                                    block_size, q.dtype, sinks, gate)
     T = q.shape[0]
     dt = q.dtype
     out = torch.empty(T, H, C, dtype=dt, device=q.device)
@@ -383,6 +414,7 @@ def latent_attention(q_abs: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, 
     args = (_p(q_abs, dt, "q_abs"), _p(q), _p(cache, dt, "cache"), _p(block_tables, I32, "block_tables"),
             block_tables.shape[1], _p(tok_seq, I32), _p(positions, I32), T, C, R, H, Dn, int(window), float(scale),
             block_size)
+    gp, ldg = (gate.data_ptr(), gate.stride(0)) if gate is not None else (0, 0)
     if LATENT_MFMA and dt == BF16 and nat.latent_mfma_ok(C, R, Dn):
         cap = block_tables.shape[1] * block_size
         bound = min(max_keys or cap, window or cap, cap)
@@ -394,9 +426,9 @@ def latent_attention(q_abs: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, 
             pml = torch.empty(T * HP * ns * 2, dtype=F32, device=q.device)
         nseq = cu_q.shape[0] - 1 if cu_q is not None else 0
         nat.latent_attention_mfma(out.data_ptr(), _p(pacc), _p(pml), *args, ns, _p(cu_q, I32, "cu_q"), nseq,
-                                  int(max_qlen), _p(sinks), -1)
+                                  int(max_qlen), _p(sinks), gp, ldg, -1)
     else:
-        nat.latent_attention(out.data_ptr(), *args, _f32(dt), _p(sinks), -1)
+        nat.latent_attention(out.data_ptr(), *args, _f32(dt), _p(sinks), gp, ldg, -1)
     return out
 
 
@@ -631,14 +663,17 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
     k (B) and q (C) (``groups`` D each; head h uses group h // (H / groups)); ``aux`` fp32 [T, lda] holds f (the step
     size logits, H) and g (the output gate, H V) at ``cols``; ``head_params`` fp32 [3, H] = -exp(A_log), dt_bias, skip.
     dt = softplus(f + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T; y = (S^T C + skip x) silu(g), returned in fp32
-    without a norm (``normw`` None, ``out_dtype`` fp32)."""
-    if proj.dtype != F32 or state.dtype != F32:
+    without a norm (``normw`` None, ``out_dtype`` fp32).
+    SCAN_DECAY (linear attention under a constant decay per head): ``proj`` in fp32 or bf16 holds q, k (``groups`` D each;
+    head h uses group h // (H / groups)) and v (H V) before their activation; ``head_params`` fp32 [H] are the decays.
+    S <- decay S + silu(k) silu(v)^T; y = S^T silu(q), returned in fp32 without a norm."""
+    if (proj.dtype != F32 and not (kind == SCAN_DECAY and proj.dtype == BF16)) or state.dtype != F32:
         raise TypeError("the recurrence's inputs and state are fp32")
     if proj.dim() != 2 or proj.stride(1) != 1:
         raise ValueError("gated_scan: projected rows must be contiguous")
     need = {SCAN_HGRN2: ("q", "f", "v"), SCAN_MLSTM: ("q", "k", "v", "i", "f", "g"),
-            SCAN_SSD: ("q", "k", "v", "f", "g")}[kind]
-    G = int(groups) if kind == SCAN_SSD else H
+            SCAN_SSD: ("q", "k", "v", "f", "g"), SCAN_DECAY: ("q", "k", "v")}[kind]
+    G = int(groups) if kind in (SCAN_SSD, SCAN_DECAY) else H
     width = {"q": G * D, "k": G * D, "v": H * V, "g": H * V, "i": H, "f": H * D if kind == SCAN_HGRN2 else H}
     if kind == SCAN_SSD:
         if aux is None or head_params is None or G <= 0 or H % G:
@@ -649,6 +684,13 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
             raise TypeError("gated_scan: head_params is contiguous fp32 [3, H]")
         if out_dtype != F32:
             raise TypeError("gated_scan: SCAN_SSD returns fp32")
+    if kind == SCAN_DECAY:
+        if head_params is None or G <= 0 or H % G:
+            raise ValueError("gated_scan: SCAN_DECAY needs head_params and groups that divide the heads")
+        if head_params.dtype != F32 or head_params.shape != (H,) or not head_params.is_contiguous():
+            raise TypeError("gated_scan: the decays are contiguous fp32 [H]")
+        if out_dtype != F32:
+            raise TypeError("gated_scan: SCAN_DECAY returns fp32")
     for key in need:
         src = aux if kind == SCAN_SSD and key in ("f", "g") else proj
         if cols[key] < 0 or cols[key] + width[key] > src.shape[1]:
@@ -667,10 +709,11 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
     Lc = (SCAN_CHUNK if T >= SCAN_CHUNK_MIN else 0) if chunk is None else int(chunk)
     ws = torch.empty(_native().gated_scan_workspace(T, nseq, H, D, V, Lc), dtype=F32, device=proj.device) if Lc > 0 \
         else None
-    _native().gated_scan(out.data_ptr(), _p(proj), proj.stride(0), kind, c("q"), c("k"), c("v"), c("i"), c("f"), c("g"),
+    _native().gated_scan(out.data_ptr(), proj.data_ptr(), proj.stride(0), kind, c("q"), c("k"), c("v"), c("i"), c("f"), c("g"),
                          _p(fbias, out_dtype, "fbias"), _p(ibias, out_dtype, "ibias"), _p(lower, out_dtype, "lower"),
                          _p(normw, out_dtype, "normw"), _p(state), _p(cu_q, I32), _p(seq_slots, I32),
-                         _p(positions, I32), nseq, H, D, V, float(eps), float(cap), _f32(out_dtype), T, Lc, _p(ws),
+                         _p(positions, I32), nseq, H, D, V, float(eps), float(cap),
+                         _f32(proj.dtype if kind == SCAN_DECAY else out_dtype), T, Lc, _p(ws),
                          aux.data_ptr() if aux is not None else 0, aux.stride(0) if aux is not None else 0,
                          _p(head_params), H // G, -1)
     return out
