@@ -196,6 +196,11 @@ int k8s_gated_scan(void* out, const void* proj, long ld, int kind, int cq, int c
                    float cap, int f32, int T, int Lc, float* ws, const float* aux, long ldaux, const float* hpar, int R,
                    hipStream_t s);
 long long k8s_gated_scan_workspace(int T, int nseq, int H, int D, int V, int Lc);
+int k8s_decay_scan_ok(int D, int V);
+long long k8s_decay_scan_workspace(int T, int nseq, int H, int D, int V);
+int k8s_decay_scan(float* out, const void* proj, long ld, int cq, int ck, int cv, const float* decay, float* state,
+                   const int* cu_q, const int* seq_slots, const int* positions, int nseq, int H, int D, int V, int R,
+                   int T, void* ws, hipStream_t s);
 int k8s_moe_align(int* sorted_tok, int* pos_of_pair, int* seg, int* tiles, int ntiles, const int* topk_idx, int P,
                   int top, int E, int BM, hipStream_t s);
 int k8s_moe_combine(void* z, const void* D, const int* pos, const float* w, const void* shared, const float* logits,
@@ -630,6 +635,16 @@ PYBIND11_MODULE(K8S_MODULE_NAME, m) {
   });
   m.def("gated_scan_workspace", [](int T, int nseq, int H, int D, int V, int Lc) {
     return k8s_gated_scan_workspace(T, nseq, H, D, V, Lc);
+  });
+  m.def("decay_scan_ok", [](int D, int V) { return k8s_decay_scan_ok(D, V) != 0; });
+  m.def("decay_scan_workspace", [](int T, int nseq, int H, int D, int V) {
+    return k8s_decay_scan_workspace(T, nseq, H, D, V);
+  });
+  m.def("decay_scan", [](uintptr_t out, uintptr_t proj, long ld, int cq, int ck, int cv, uintptr_t decay, uintptr_t state,
+                         uintptr_t cu_q, uintptr_t seq_slots, uintptr_t positions, int nseq, int H, int D, int V, int R,
+                         int T, uintptr_t ws, int64_t s) {
+    check(k8s_decay_scan(P<float>(out), P(proj), ld, cq, ck, cv, P<float>(decay), P<float>(state), P<int>(cu_q),
+                         P<int>(seq_slots), P<int>(positions), nseq, H, D, V, R, T, P(ws), S(s)), "decay_scan");
   });
   m.def("moe_align", [](uintptr_t sorted_tok, uintptr_t pos, uintptr_t seg, uintptr_t tiles, int ntiles,
                         uintptr_t topk_idx, int P_, int top, int E, int BM, int64_t s) {

@@ -379,7 +379,8 @@ class KatidraModel(StreamModel):
         H, D, V = m.heads, m.dim, m.vdim
         proj = sm.linear(h, w.w_in)                                        # [T, q | k | v | gate]
         y = sm.gated_scan(proj, sm.SCAN_DECAY, w.cols, None, self.states[cache], b["cu_q"], b["seq_slots"],
-                          b["positions"], H, D, V, self.cfg.rms_eps, F32, head_params=w.decay, groups=H)
+                          b["positions"], H, D, V, self.cfg.rms_eps, F32, head_params=w.decay, groups=H,
+                          max_qlen=b.get("max_qlen", 0))
         y = sm.norm_mix(y, w.norm, None, None, self.cfg.rms_eps, out_dtype=self.dtype,
                         gate=proj[:, w.cols["g"]:w.cols["g"] + H * V])
         return sm.linear(y, w.o)

@@ -1,7 +1,7 @@
 """Ops of models with an fp32 residual stream, recurrent / windowed- or latent-attention mixers and mixtures of experts.
 
 Same dispatch rule as the rest of :mod:`..ops`: CUDA (= HIP) tensors always run the gfx950 kernels
-(``stream32.hip``, ``mixers.hip``, ``window_attn.hip``, ``gated_scan.hip``, ``delta_scan.hip``, ``moe.hip``) and raise when the extension is missing; CPU tensors run the fp32
+(``stream32.hip``, ``mixers.hip``, ``window_attn.hip``, ``gated_scan.hip``, ``decay_scan.hip``, ``delta_scan.hip``, ``moe.hip``) and raise when the extension is missing; CPU tensors run the fp32
 reference in :mod:`.reference` (the CPU test-suite).  Every op takes bf16 or true-fp32 activations / weights (the
 ``f32`` flag of the kernels); what a design computes in fp32 regardless (residual sum, recurrent state, decays, router,
 attention scores) is fp32 in both.
@@ -646,6 +646,8 @@ def gated_scan_record(kind: int, D: int, V: int) -> int:
 # over chunks); shorter ones (decoding, short portions) as one workgroup per sequence.
 SCAN_CHUNK = int(os.environ.get("K8S_SCAN_CHUNK", "64"))
 SCAN_CHUNK_MIN = int(os.environ.get("K8S_SCAN_CHUNK_MIN", "256"))
+# SCAN_DECAY in bf16 with a portion of at least this many tokens runs on the matrix cores (0: never)
+DECAY_MFMA_MIN = int(os.environ.get("K8S_DECAY_MFMA_MIN", "32"))
 
 
 def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, state: torch.Tensor, cu_q: torch.Tensor,
@@ -653,7 +655,7 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
                fbias: Optional[torch.Tensor] = None, ibias: Optional[torch.Tensor] = None,
                lower: Optional[torch.Tensor] = None, cap: float = 0.0, chunk: Optional[int] = None,
                aux: Optional[torch.Tensor] = None, head_params: Optional[torch.Tensor] = None,
-               groups: int = 0) -> torch.Tensor:
+               groups: int = 0, max_qlen: int = 0) -> torch.Tensor:
     """A gated linear recurrence with a matrix state per head over a varlen batch; ``proj`` fp32 [T, ld] is the fused
     input projection with its parts at the column offsets ``cols``; ``state`` [slots, H, record] fp32 is updated in
     place (a portion at position 0 starts from zero).  Returns the normed (and, SCAN_MLSTM, gated) outputs [T, H V].
@@ -666,7 +668,9 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
     without a norm (``normw`` None, ``out_dtype`` fp32).
     SCAN_DECAY (linear attention under a constant decay per head): ``proj`` in fp32 or bf16 holds q, k (``groups`` D each;
     head h uses group h // (H / groups)) and v (H V) before their activation; ``head_params`` fp32 [H] are the decays.
-    S <- decay S + silu(k) silu(v)^T; y = S^T silu(q), returned in fp32 without a norm."""
+    S <- decay S + silu(k) silu(v)^T; y = S^T silu(q), returned in fp32 without a norm.  ``max_qlen``: the longest
+    portion; bf16 portions of at least DECAY_MFMA_MIN tokens whose sizes fit run on the matrix cores (decay_scan.hip),
+    anything else, or with ``chunk`` given, as the other kinds do."""
     if (proj.dtype != F32 and not (kind == SCAN_DECAY and proj.dtype == BF16)) or state.dtype != F32:
         raise TypeError("the recurrence's inputs and state are fp32")
     if proj.dim() != 2 or proj.stride(1) != 1:
@@ -706,6 +710,14 @@ def gated_scan(proj: torch.Tensor, kind: int, cols: dict, normw: torch.Tensor, s
     out = torch.empty(T, H * V, dtype=out_dtype, device=proj.device)
     c = lambda key: int(cols.get(key, 0))
     nseq = cu_q.shape[0] - 1
+    if (kind == SCAN_DECAY and chunk is None and proj.dtype == BF16 and 0 < DECAY_MFMA_MIN <= max_qlen
+            and _native().decay_scan_ok(D, V) and proj.data_ptr() % 16 == 0
+            and not any(n % 8 for n in (proj.stride(0), c("q"), c("k"), c("v")))):
+        ws = torch.empty(_native().decay_scan_workspace(T, nseq, H, D, V), dtype=torch.uint8, device=proj.device)
+        _native().decay_scan(out.data_ptr(), proj.data_ptr(), proj.stride(0), c("q"), c("k"), c("v"), _p(head_params),
+                             _p(state), _p(cu_q, I32), _p(seq_slots, I32), _p(positions, I32), nseq, H, D, V, H // G, T,
+                             _p(ws), -1)
+        return out
     Lc = (SCAN_CHUNK if T >= SCAN_CHUNK_MIN else 0) if chunk is None else int(chunk)
     ws = torch.empty(_native().gated_scan_workspace(T, nseq, H, D, V, Lc), dtype=F32, device=proj.device) if Lc > 0 \
         else None

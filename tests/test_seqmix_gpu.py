@@ -627,14 +627,27 @@ def test_latent_attention_interleaved_pairs_and_sinks(dt, tol, H, Dn, R, C, dims
     oc = sm.latent_attention(qabs, qc, cc, bt, tok_seq, pos, C, R, H, Dn, 0, 0.2, bs, sinks=sinks)
     assert not torch.allclose(oc.float(), sm.latent_attention(qabs, qc, cc, bt, tok_seq, pos, C, R, H, Dn, 0, 0.2, bs).float(),
                               atol=1e-2)
+    wide_gate = (torch.randn(T, H + 24) * 2).to(dt)                           # a gate per head, a slice of a projection
+    gate = wide_gate[:, 8:8 + H]
+    gg = wide_gate.to(DEV)[:, 8:8 + H]
+    gated = sm.latent_attention(qabs, qc, cc, bt, tok_seq, pos, C, R, H, Dn, 0, 0.2, bs, gate=gate)
+    want = ref.latent_attention(qabs, qc, cc, bt, tok_seq, pos, C, R, H, Dn, 0, 0.2, bs, torch.float32) \
+        * torch.sigmoid(gate.float()).unsqueeze(-1)
+    close(gated, want, 1e-2 if dt == torch.bfloat16 else 1e-6)
     for kw in ({}, {"cu_q": cu.to(DEV), "max_qlen": 27}):
         og = sm.latent_attention(qabs.to(DEV), qc.to(DEV), cc.to(DEV), bt.to(DEV), tok_seq.to(DEV), pos.to(DEV), C, R, H,
                                  Dn, 0, 0.2, bs, sinks=sinks.to(DEV), **kw)
         close(og, oc, tol)
+        og = sm.latent_attention(qabs.to(DEV), qc.to(DEV), cc.to(DEV), bt.to(DEV), tok_seq.to(DEV), pos.to(DEV), C, R, H,
+                                 Dn, 0, 0.2, bs, gate=gg, **kw)
+        close(og, gated, tol)
     few = torch.tensor([3, 20, 30], dtype=torch.long)                         # few tokens: key splits and their merge
     og = sm.latent_attention(qabs[few].to(DEV), qc[few].to(DEV), cc.to(DEV), bt.to(DEV), tok_seq[few].to(DEV),
                              pos[few].to(DEV), C, R, H, Dn, 0, 0.2, bs, 64, sinks=sinks.to(DEV))
     close(og, oc[few], tol)
+    og = sm.latent_attention(qabs[few].to(DEV), qc[few].to(DEV), cc.to(DEV), bt.to(DEV), tok_seq[few].to(DEV),
+                             pos[few].to(DEV), C, R, H, Dn, 0, 0.2, bs, 64, gate=gg[few.to(DEV)])
+    close(og, gated[few], tol)
 
 
 @pytest.mark.parametrize("dt,tol", DTYPES)
@@ -708,3 +721,127 @@ def test_latent_attention_prompt_with_long_block_tables(width):
     og = sm.latent_attention(qabs.to(DEV), q.to(DEV), cache.to(DEV), bt.to(DEV), tok_seq.to(DEV), pos.to(DEV), C, R, H, Dn,
                              0, 0.2, bs, cu_q=cu.to(DEV), max_qlen=27)
     close(og, oc, tol)
+
+
+# ----------------------------------------------------------------------------- norms of the branch, squared relu
+@pytest.mark.parametrize("dt,tol", DTYPES)
+@pytest.mark.parametrize("W", [200, 64, 1, 513, 2048, 2500, 5000])
+def test_branchnorm_squared_relu_and_gated_norm(dt, tol, W):
+    torch.manual_seed(60)
+    x, w = torch.randn(T, W) * 2, (1 + 0.3 * torch.randn(W)).to(dt)
+    for br in ((torch.randn(T, W) * 3).to(dt), torch.randn(T, W) * 1e-3):       # activation type; fp32, near eps
+        xg, xc = x.to(DEV).clone(), x.clone()
+        og = sm.branchnorm(xg, br.to(DEV), w.to(DEV), 1e-5, out_dtype=dt)
+        oc = sm.branchnorm(xc, br, w, 1e-5, out_dtype=dt)
+        assert og.dtype == dt
+        close(og, oc, tol)
+        close(xg, xc, 1e-5)
+        assert sm.branchnorm(xg, br.to(DEV), w.to(DEV), 1e-5) is None
+        sm.branchnorm(xc, br, w, 1e-5)
+        close(xg, xc, 1e-5)
+    a = (torch.randn(T, W) * 2).to(dt)
+    got = sm.act(a.to(DEV), sm.ACT_RELU2)
+    close(got, sm.act(a, sm.ACT_RELU2), tol)
+    close(got, a.float().clamp(min=0).square().to(dt), tol)
+    # a norm whose result is gated by a slice of a wider tensor, over the whole row and in groups
+    wide, y, wn = (torch.randn(T, W + 40) * 2).to(dt), torch.randn(T, W), 1 + 0.2 * torch.randn(W)
+    for groups in (1, 4 if W % 4 == 0 else 1):
+        for kind in (sm.GATE_SIGMOID, sm.GATE_SILU):
+            kw = dict(out_dtype=dt, groups=groups, gate_kind=kind)
+            og = sm.norm_mix(y.to(DEV), wn.to(DEV), None, None, 1e-5, gate=wide.to(DEV)[:, 16:16 + W], **kw)
+            close(og, sm.norm_mix(y, wn, None, None, 1e-5, gate=wide[:, 16:16 + W], **kw), tol)
+
+
+# ----------------------------------------------------------------------------- linear attention with a constant decay
+def _decay_case(dt, H, G, D, V, cu, pos, pad=16):
+    n = int(cu[-1])
+    up = lambda m: (m + pad - 1) // pad * pad
+    cols = {"q": 0, "k": up(G * D), "v": 2 * up(G * D)}
+    proj = torch.randn(n, cols["v"] + up(H * V) + pad).to(dt)
+    decay = torch.tensor([(0.999, 0.5, 1.0, 0.97, 1e-3, 0.9)[h % 6] for h in range(H)])
+    return proj, cols, decay, torch.randn(4, H, D * V) * 0.5
+
+
+@pytest.mark.parametrize("dt", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,G,D,V", [(4, 2, 16, 24), (3, 3, 40, 56), (3, 1, 100, 5), (2, 2, 128, 64), (6, 3, 64, 128),
+                                     (1, 1, 256, 200), (5, 5, 7, 70), (1, 1, 1, 1)])
+def test_decay_scan(dt, H, G, D, V):
+    """One workgroup per sequence and three passes over chunks, in both input types (the inputs are the same rounded
+    numbers for the reference, and everything after them is fp32)."""
+    torch.manual_seed(61)
+    cu, pos, slots, _ = batch()
+    proj, cols, decay, state = _decay_case(dt, H, G, D, V, cu, pos, pad=3)
+    sc, sg = state.clone(), state.to(DEV).clone()
+    args = lambda d, s: (proj.to(d), sm.SCAN_DECAY, cols, None, s, cu.to(d), slots.to(d), pos.to(d), H, D, V, 1e-6,
+                         torch.float32)
+    kw = lambda d: dict(head_params=decay.to(d), groups=G)
+    oc = sm.gated_scan(*args("cpu", sc), **kw("cpu"))
+    og = sm.gated_scan(*args(DEV, sg), **kw(DEV))
+    assert og.dtype == torch.float32
+    close(og, oc, 2e-5)
+    close(sg, sc, 1e-5)
+    assert torch.equal(sg[1].cpu(), state[1])                                  # the empty sequence's slot
+    for chunk in (4, 7, 16, 64):                       # three passes over chunks: same outputs, same final states
+        s2 = state.to(DEV).clone()
+        o2 = sm.gated_scan(*args(DEV, s2), chunk=chunk, **kw(DEV))
+        close(o2, oc, 2e-5)
+        close(s2, sc, 1e-5)
+
+
+@pytest.mark.parametrize("lens", [(9, 1, 0, 27), (64, 65, 63, 1), (200, 0, 128, 7), (2, 2, 2, 2), (600, 1, 1, 0)])
+@pytest.mark.parametrize("H,G,D,V", [(4, 2, 16, 24), (3, 3, 40, 56), (2, 1, 128, 128), (6, 3, 64, 8), (2, 2, 8, 248),
+                                     (1, 1, 96, 160), (5, 5, 32, 64), (3, 3, 72, 80)])
+def test_decay_scan_on_the_matrix_cores(monkeypatch, H, G, D, V, lens):
+    """Chunks as products of tiles against the step-by-step reference: several sequences of unequal length, from zero
+    and from carried states, chunks that are full, cut short or a single token.  The kernel rounds q, k and v to bf16 after
+    their activation: it follows the reference closely when that rounds them too, and within bf16 when it does not."""
+    torch.manual_seed(62)
+    cu = torch.tensor([0] + list(torch.tensor(lens).cumsum(0)), dtype=torch.int32)
+    p0 = (0, 5, 0, 130)                                                        # two sequences start, two go on
+    pos = torch.cat([torch.arange(p, p + n) for p, n in zip(p0, lens)]).int()
+    slots = torch.tensor([2, 0, 1, 3], dtype=torch.int32)
+    proj, cols, decay, state = _decay_case(torch.bfloat16, H, G, D, V, cu, pos)
+    sc, sg = state.clone(), state.to(DEV).clone()
+    args = lambda d, s: (proj.to(d), sm.SCAN_DECAY, cols, None, s, cu.to(d), slots.to(d), pos.to(d), H, D, V, 1e-6,
+                         torch.float32)
+    oc = sm.gated_scan(*args("cpu", sc), head_params=decay, groups=G)
+    calls = []
+    nat = sm._native()
+
+    class Spy:
+        def __getattr__(self, name):
+            if name == "decay_scan":
+                calls.append(name)
+            return getattr(nat, name)
+
+    real, sm._native = sm._native, lambda: Spy()
+    try:
+        og = sm.gated_scan(*args(DEV, sg), head_params=decay.to(DEV), groups=G, max_qlen=max(max(lens), 32))
+    finally:
+        sm._native = real
+    assert calls                                                               # not the per-token kernel
+    assert torch.isfinite(og).all()
+    for h in range(H):                                  # per head: fast and slow decays have outputs of other sizes
+        a, b = og.cpu().view(-1, H, V)[:, h], oc.view(-1, H, V)[:, h]
+        close(a, b, 2e-2)
+        close(sg.cpu()[:, h], sc[:, h], 2e-2)
+    for i, n in enumerate(lens):                        # a sequence without tokens leaves its slot alone
+        if n == 0:
+            assert torch.equal(sg[int(slots[i])].cpu(), state[int(slots[i])])
+    silu = torch.nn.functional.silu
+    with monkeypatch.context() as m:
+        m.setattr(torch.nn.functional, "silu", lambda z: silu(z).bfloat16().float())
+        sr = state.clone()
+        rounded = sm.gated_scan(*args("cpu", sr), head_params=decay, groups=G)
+    for h in range(H):
+        for a, b in ((og.cpu().view(-1, H, V)[:, h], rounded.view(-1, H, V)[:, h]), (sg.cpu()[:, h], sr[:, h])):
+            assert (a - b).pow(2).mean().sqrt() < 3e-4 * b.pow(2).mean().sqrt(), h
+    # inputs whose activations are exact in bf16 leave only the two-term rounding of weights, scores and state
+    exact = torch.where(proj > 0, torch.full_like(proj, 40.0), torch.full_like(proj, -200.0))   # silu: 40 and 0
+    s1, s2 = state.clone(), state.to(DEV).clone()
+    a1 = lambda d, s: (exact.to(d), *args(d, s)[1:])
+    o1 = sm.gated_scan(*a1("cpu", s1), head_params=decay, groups=G)
+    o2 = sm.gated_scan(*a1(DEV, s2), head_params=decay.to(DEV), groups=G, max_qlen=max(max(lens), 32))
+    for h in range(H):
+        close(o2.cpu().view(-1, H, V)[:, h], o1.view(-1, H, V)[:, h], 5e-5)
+        close(s2.cpu()[:, h], s1[:, h], 5e-5)
