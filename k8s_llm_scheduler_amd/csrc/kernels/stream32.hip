@@ -89,36 +89,56 @@ __global__ __launch_bounds__(256) void postnorm_kernel(float* __restrict__ x, co
   }
 }
 
+// Four consecutive elements as fp32, and back; pointers aligned to the four elements.
+template <typename T> __device__ __forceinline__ f32x4 ldf4(const T* p);
+template <> __device__ __forceinline__ f32x4 ldf4<float>(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+template <> __device__ __forceinline__ f32x4 ldf4<bf16_t>(const bf16_t* p) {
+  const uint2 u = *reinterpret_cast<const uint2*>(p);
+  return f32x4{lo_bf(u.x), hi_bf(u.x), lo_bf(u.y), hi_bf(u.y)};
+}
+template <typename T> __device__ __forceinline__ void stf4(T* p, f32x4 v);
+template <> __device__ __forceinline__ void stf4<float>(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+template <> __device__ __forceinline__ void stf4<bf16_t>(bf16_t* p, f32x4 v) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
+}
+
 // Norm of a sublayer's output ahead of the sum: x[t] += branch[t] / sqrt(mean(branch[t]^2) + eps) * w, in fp32; `out`
 // (optional) receives the new row in the activation type, for the sublayer that reads the stream next.  One workgroup
-// per row; NR > 0: the row's branch values stay in registers between the two passes (W <= 256 NR), else they are read
-// again.
-template <typename TB, typename TA, int NR>
+// per row.  NV > 0 (W % 4 == 0, W <= 1024 NV): everything a thread needs is loaded as vectors ahead of the reduction and
+// stays in registers; else the row is read again after it.
+template <typename TB, typename TA, int NV>
 __global__ __launch_bounds__(256) void branchnorm_kernel(float* __restrict__ x, const TB* __restrict__ branch,
                                                          const TA* __restrict__ w, float eps, TA* __restrict__ out,
                                                          int W) {
   __shared__ float red[16];
   const size_t base = (size_t)blockIdx.x * W;
   float ss = 0.f;
-  if constexpr (NR > 0) {
-    float v[NR], xv[NR];
+  if constexpr (NV > 0) {
+    const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
+    f32x4 v[NV], xv[NV], wv[NV];
 #pragma unroll
-    for (int n = 0; n < NR; ++n) {
-      const int i = threadIdx.x + 256 * n;
-      v[n] = i < W ? ldf(branch, base + i) : 0.f;
-      xv[n] = i < W ? x[base + i] : 0.f;
+    for (int n = 0; n < NV; ++n) {
+      const int i = 4 * (threadIdx.x + 256 * n);
+      const bool in = i < W;
+      v[n] = in ? ldf4(branch + base + i) : zero;
+      xv[n] = in ? ldf4(x + base + i) : zero;
+      wv[n] = in ? ldf4(w + i) : zero;
     }
 #pragma unroll
-    for (int n = 0; n < NR; ++n) ss += v[n] * v[n];
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += v[n][e] * v[n][e];
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)W + eps);
 #pragma unroll
-    for (int n = 0; n < NR; ++n) {
-      const int i = threadIdx.x + 256 * n;
+    for (int n = 0; n < NV; ++n) {
+      const int i = 4 * (threadIdx.x + 256 * n);
       if (i >= W) continue;
-      const float y = fmaf(v[n] * inv, ldf(w, i), xv[n]);
-      x[base + i] = y;
-      if (out != nullptr) stf(out, base + i, y);
+      f32x4 y;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = fmaf(v[n][e] * inv, wv[n][e], xv[n][e]);
+      stf4(x + base + i, y);
+      if (out != nullptr) stf4(out + base + i, y);
     }
   } else {
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
@@ -153,10 +173,27 @@ __global__ void gate_mul_kernel(TA* __restrict__ out, const TY* __restrict__ y, 
 // 6 limit * tanh(x / limit), 7 relu(x)^2: elementwise on [T, F].
 // Elementwise kinds take a factor per row: logical row i is row row_map[i] (or i) and its input is multiplied by
 // row_scale[i] before the function (experts whose router weight scales their input).
+__device__ __forceinline__ float act_elem(float v, int kind, float limit) {
+  return kind == 2   ? tanhf(v)
+         : kind == 3 ? v / (1.f + expf(-v))
+         : kind == 4 ? 0.5f * v * (1.f + erff(v * 0.7071067811865476f))
+         : kind == 7 ? (v > 0.f ? v * v : 0.f)
+                     : limit * tanhf(v / limit);
+}
 template <typename TA>
 __global__ void act_kernel(TA* __restrict__ out, const TA* __restrict__ x, int T, int F, int kind, float limit,
                            float alpha, const float* __restrict__ row_scale, const int* __restrict__ row_map) {
   const size_t n = (size_t)T * F;
+  if (kind >= 2 && kind != 5 && row_scale == nullptr && row_map == nullptr && n % 4 == 0 &&
+      ((uintptr_t)x | (uintptr_t)out) % (4 * sizeof(TA)) == 0) {   // no row index needed
+    for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n / 4; i += (size_t)gridDim.x * blockDim.x) {
+      f32x4 v = ldf4(x + 4 * i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = act_elem(v[e], kind, limit);
+      stf4(out + 4 * i, v);
+    }
+    return;
+  }
   for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / F, c = i - t * F;
     float y;
@@ -165,11 +202,7 @@ __global__ void act_kernel(TA* __restrict__ out, const TA* __restrict__ x, int T
       if (row_map != nullptr) o = (size_t)row_map[t] * F + c;
       float v = ldf(x, o);
       if (row_scale != nullptr) v *= row_scale[t];
-      y = kind == 2   ? tanhf(v)
-          : kind == 3 ? v / (1.f + expf(-v))
-          : kind == 4 ? 0.5f * v * (1.f + erff(v * 0.7071067811865476f))
-          : kind == 7 ? (v > 0.f ? v * v : 0.f)
-                      : limit * tanhf(v / limit);
+      y = act_elem(v, kind, limit);
     } else {
       float g = ldf(x, t * 2 * F + c), u = ldf(x, t * 2 * F + F + c);
       if (kind == 0) {
@@ -198,6 +231,49 @@ __device__ __forceinline__ float gate_of(const TO* gate, size_t i, int gkind) {
   const float g = ldf(gate, i), s = 1.f / (1.f + expf(-g));
   return gkind == 1 ? g * s : s;
 }
+// The single-input form without groups for rows of whole vectors (W % 4 == 0, W <= 1024 NV, every pointer and stride
+// aligned to four elements): all loads ahead of the reduction, everything in registers.
+template <typename TA, typename TO, int NV>
+__global__ __launch_bounds__(256) void norm_row_kernel(TO* __restrict__ out, const TA* __restrict__ a, long lda,
+                                                       const TA* __restrict__ wa, float eps, float ca, int W,
+                                                       const TO* __restrict__ gate, long ldg, int gkind) {
+  __shared__ float red[16];
+  const TA* ar = a + (size_t)blockIdx.x * lda;
+  const TO* gr = gate != nullptr ? gate + (size_t)blockIdx.x * ldg : nullptr;
+  const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
+  f32x4 v[NV], wv[NV], gv[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int n = 0; n < NV; ++n) {
+    const int i = 4 * (threadIdx.x + 256 * n);
+    const bool in = i < W;
+    v[n] = in ? ldf4(ar + i) : zero;
+    wv[n] = in ? ldf4(wa + i) : zero;
+    gv[n] = in && gr != nullptr ? ldf4(gr + i) : zero;
+  }
+#pragma unroll
+  for (int n = 0; n < NV; ++n)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += v[n][e] * v[n][e];
+  ss = block_sum(ss, red);
+  const float inv = ca / sqrtf(ss / (float)W + eps);
+#pragma unroll
+  for (int n = 0; n < NV; ++n) {
+    const int i = 4 * (threadIdx.x + 256 * n);
+    if (i >= W) continue;
+    f32x4 y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      y[e] = v[n][e] * inv * wv[n][e];
+      if (gr != nullptr) {
+        const float s = 1.f / (1.f + expf(-gv[n][e]));
+        y[e] *= gkind == 1 ? gv[n][e] * s : s;
+      }
+    }
+    stf4(out + (size_t)blockIdx.x * W + i, y);
+  }
+}
+
 template <typename TA, typename TO>
 __global__ __launch_bounds__(256) void norm_mix_kernel(TO* __restrict__ out, const TA* __restrict__ a, long lda,
                                                        const TA* __restrict__ wa, const TA* __restrict__ b,
@@ -457,10 +533,26 @@ extern "C" int k8s_norm_mix(void* out, const void* a, long lda, const void* wa, 
 #define K8S_NM(TA, TO)                                                                                             \
   norm_mix_kernel<TA, TO><<<T, 256, 0, s>>>((TO*)out, (const TA*)a, lda, (const TA*)wa, (const TA*)b, (const TA*)wb, \
                                             eps, ca, cb, W, groups, (const TO*)gate, ldg, gkind)
-  if (in_f32 && out_f32) K8S_NM(float, float);
-  else if (in_f32) K8S_NM(float, bf16_t);
-  else if (out_f32) K8S_NM(bf16_t, float);
-  else K8S_NM(bf16_t, bf16_t);
+#define K8S_NR(TA, TO, NV) \
+  norm_row_kernel<TA, TO, NV><<<T, 256, 0, s>>>((TO*)out, (const TA*)a, lda, (const TA*)wa, eps, ca, W, (const TO*)gate, \
+                                                ldg, gkind)
+#define K8S_NM_T(TA, TO)                                                                              \
+  do {                                                                                                \
+    const bool vec = b == nullptr && groups == 1 && W % 4 == 0 && W <= 8192 && lda % 4 == 0 &&        \
+                     (uintptr_t)a % (4 * sizeof(TA)) == 0 && (uintptr_t)wa % (4 * sizeof(TA)) == 0 && \
+                     (uintptr_t)out % (4 * sizeof(TO)) == 0 && (uintptr_t)gate % (4 * sizeof(TO)) == 0 && ldg % 4 == 0; \
+    if (!vec) K8S_NM(TA, TO);                                                                         \
+    else if (W <= 1024) K8S_NR(TA, TO, 1);                                                            \
+    else if (W <= 2048) K8S_NR(TA, TO, 2);                                                            \
+    else if (W <= 4096) K8S_NR(TA, TO, 4);                                                            \
+    else K8S_NR(TA, TO, 8);                                                                           \
+  } while (0)
+  if (in_f32 && out_f32) K8S_NM_T(float, float);
+  else if (in_f32) K8S_NM_T(float, bf16_t);
+  else if (out_f32) K8S_NM_T(bf16_t, float);
+  else K8S_NM_T(bf16_t, bf16_t);
+#undef K8S_NM_T
+#undef K8S_NR
 #undef K8S_NM
   return (int)hipGetLastError();
 }
@@ -483,14 +575,17 @@ extern "C" int k8s_branchnorm(float* x, const void* branch, const void* w, float
                               int branch_f32, int f32, hipStream_t s) {
   if (T <= 0) return 0;
   if (W <= 0 || x == nullptr || branch == nullptr || w == nullptr || (f32 && !branch_f32)) return -1;
-#define K8S_BN(TB, TA, NR) \
-  branchnorm_kernel<TB, TA, NR><<<T, 256, 0, s>>>(x, (const TB*)branch, (const TA*)w, eps, (TA*)out, W)
-#define K8S_BN_T(TB, TA)                       \
-  do {                                         \
-    if (W <= 512) K8S_BN(TB, TA, 2);           \
-    else if (W <= 2048) K8S_BN(TB, TA, 8);     \
-    else if (W <= 4096) K8S_BN(TB, TA, 16);    \
-    else K8S_BN(TB, TA, 0);                    \
+#define K8S_BN(TB, TA, NV) \
+  branchnorm_kernel<TB, TA, NV><<<T, 256, 0, s>>>(x, (const TB*)branch, (const TA*)w, eps, (TA*)out, W)
+#define K8S_BN_T(TB, TA)                                                                                   \
+  do {                                                                                                     \
+    const bool vec = W % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)branch % (4 * sizeof(TB)) == 0 &&  \
+                     (uintptr_t)w % (4 * sizeof(TA)) == 0 && (uintptr_t)out % (4 * sizeof(TA)) == 0;       \
+    if (!vec || W > 8192) K8S_BN(TB, TA, 0);                                                               \
+    else if (W <= 1024) K8S_BN(TB, TA, 1);                                                                 \
+    else if (W <= 2048) K8S_BN(TB, TA, 2);                                                                 \
+    else if (W <= 4096) K8S_BN(TB, TA, 4);                                                                 \
+    else K8S_BN(TB, TA, 8);                                                                                \
   } while (0)
   if (f32) K8S_BN_T(float, float);
   else if (branch_f32) K8S_BN_T(float, bf16_t);
@@ -526,7 +621,8 @@ extern "C" int k8s_act(void* out, const void* x, int T, int F, int kind, float l
   if (kind < 0 || kind > 7 || (gated && (row_scale != nullptr || row_map != nullptr)) || (kind == 6 && !(limit > 0.f)))
     return -1;
   const size_t n = (size_t)T * F;
-  const int blocks = (int)((n + 255) / 256 > 4096 ? 4096 : (n + 255) / 256);
+  const size_t nt = gated ? n : (n + 3) / 4;   // elementwise kinds: four elements per thread
+  const int blocks = (int)((nt + 255) / 256 > 4096 ? 4096 : (nt + 255) / 256);
   if (f32) act_kernel<float><<<blocks, 256, 0, s>>>((float*)out, (const float*)x, T, F, kind, limit, alpha,
                                                     row_scale, row_map);
   else act_kernel<bf16_t><<<blocks, 256, 0, s>>>((bf16_t*)out, (const bf16_t*)x, T, F, kind, limit, alpha,

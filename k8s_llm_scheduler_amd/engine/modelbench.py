@@ -1,7 +1,8 @@
 """Prefill and decode throughput of the registered model designs at equal layer sizes (``bench.py --model-bench``).
 
 For every size a Putulorn (dense feed-forwards), a Putulorn with experts, a Rupatar (experts in every layer), a Nukizen
-(dense feed-forward beside every mixer), a Semanex (dense feed-forward after every mixer) and a Llama of the same width, depth, feed-forward / expert size and vocabulary are built with random weights and driven through the
+(dense feed-forward beside every mixer), a Semanex and a Katidra (dense feed-forward after every mixer) and a Llama of
+the same width, depth, feed-forward / expert size and vocabulary are built with random weights and driven through the
 same engine entry points:
 
 * prefill: one whole prompt of ``T`` tokens in one step (``LLMEngine.replay_step``, the varlen forward), tokens/s;
@@ -23,13 +24,20 @@ VOCAB = 32768
 
 
 def _register(width: int) -> Dict[str, str]:
-    from ..models import nukizen, putulorn, rupatar, semanex
+    from ..models import katidra, nukizen, putulorn, rupatar, semanex
     from ..models.config import PRESETS, LlamaConfig
 
     pairs, ff, wd, heads, eff, experts = SIZES[width]
     names = {"putulorn-dense": f"putulorn-w{width}-dense", "putulorn-moe": f"putulorn-w{width}-moe",
              "rupatar": f"rupatar-w{width}", "nukizen": f"nukizen-w{width}", "semanex": f"semanex-w{width}",
-             "llama": f"llama-w{width}"}
+             "katidra": f"katidra-w{width}", "llama": f"llama-w{width}"}
+    # Katidra: pairs of a lightning layer (128 x 128 states, heads filling the width) and a latent attention shaped like
+    # Putulorn's (rank 512 + 64 rotated, 128-wide heads, window 1024) with a query latent of 3 / 4 of the width, the
+    # feed-forward size of the Putulorn-dense layers; every layer has weights of its own
+    katidra.PRESETS[names["katidra"]] = katidra.preset(
+        names["katidra"], width, VOCAB, ("lightning", "latent_attention") * pairs, heads=heads, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, q_rank=width * 3 // 4, window=1024, scan_heads=width // 128, scan_dim=128, scan_vdim=128,
+        ff=ff)
     # Semanex: 2 x pairs layers in the order latent, latent, parallel (capped attention + state-space recurrence),
     # latent; latent attention shaped like Putulorn's (rank 512 + 64 rotated, 128-wide heads) with a query latent of
     # 3 / 4 of the width, the side attention like Rupatar's (4 query heads per key head, 128-wide), recurrent heads of
