@@ -68,9 +68,10 @@ XgmiComm::XgmiComm(int world, int rank, long long slot_bytes, int blocks, double
 XgmiComm::~XgmiComm() {
   for (int i = 0; i < world_; ++i)
     if (mapped_[i] && bases_[i]) (void)hipIpcCloseMemHandle(bases_[i]);
-  if (region_) (void)hipFree(region_);
+  // region_ and fused_state_ are uncached device memory that kernels have read: they stay allocated until the process
+  // ends, since later allocations that take such freed memory over have held wrong values.  A process makes one or two
+  // communicators, so what stays is bounded.
   if (counters_) (void)hipFree(counters_);
-  if (fused_state_) (void)hipFree(fused_state_);
   if (host_err_) (void)hipHostFree(host_err_);
 }
 

@@ -187,8 +187,10 @@ def test_xgmi_two_ranks_one_gpu():
                 if any(p.exitcode not in (None, 0) for p in procs):
                     break
     finally:
+        # a rank that failed leaves the other one waiting for it: end that one now, so that the reason is reported
+        done = len(got) == WORLD and all(v[0] == "ok" for v in got.values())
         for p in procs:
-            p.join(120)
+            p.join(30 if done else 2)
             if p.is_alive():
                 p.kill()
     fails = {r: v[1] for r, v in got.items() if v[0] != "ok"}
