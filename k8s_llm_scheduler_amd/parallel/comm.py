@@ -105,9 +105,9 @@ class TPGroup:
                 self._log_ar("rccl", nbytes)
                 self.rccl_calls += 1
                 self.rccl.all_reduce(t.data_ptr(), t.data_ptr(), t.numel(), _DT[t.dtype], 0, -1)
-            elif self.backend == "gloo" and t.dtype == torch.bfloat16:
+            elif self.backend == "gloo" and (t.is_cuda or t.dtype == torch.bfloat16):
                 self._log_ar("gloo", nbytes)
-                f = t.float()
+                f = (t.float() if t.dtype == torch.bfloat16 else t).cpu()   # gloo exchanges host memory only
                 dist.all_reduce(f, group=self.group)
                 t.copy_(f)
             else:
@@ -148,7 +148,10 @@ class TPGroup:
             self.rccl_calls += 1
             self.rccl.all_gather(t.data_ptr(), out.data_ptr(), t.numel(), _DT[t.dtype], -1)
         elif self.backend == "gloo":
-            dist.all_gather(list(out.unbind(0)), t.contiguous(), group=self.group)
+            host = torch.empty(out.shape, dtype=t.dtype) if t.is_cuda else out   # gloo exchanges host memory only
+            dist.all_gather(list(host.unbind(0)), t.cpu(), group=self.group)
+            if host is not out:
+                out.copy_(host)
         else:
             dist.all_gather_into_tensor(out, t.contiguous(), group=self.group)
         return out
@@ -186,7 +189,10 @@ class TPGroup:
 
     def broadcast_(self, t: torch.Tensor, src: int = 0) -> torch.Tensor:
         if self.world > 1:
-            dist.broadcast(t, src=self.leader + src, group=self.group)
+            host = t.cpu() if self.backend == "gloo" else t
+            dist.broadcast(host, src=self.leader + src, group=self.group)
+            if host is not t:
+                t.copy_(host)
         return t
 
     def barrier(self) -> None:
@@ -835,7 +841,7 @@ def autotune_comm(tp: TPGroup, sizes=(16384, 65536, 262144, 1 << 20, 4 << 20, 8 
     def timed(fn) -> float:
         dist.barrier(group=tp.group)
         us = _graph_time_us(fn)
-        t = torch.tensor([us], dtype=torch.float64, device=dev)
+        t = torch.tensor([us], dtype=torch.float64, device="cpu" if tp.backend == "gloo" else dev)
         dist.all_reduce(t, op=dist.ReduceOp.MAX, group=tp.group)
         return float(t[0])
 
